@@ -11,8 +11,10 @@
 //                 and of k is divided by its root mean square over its dk numbers (eps inside the root) and multiplied by a
 //                 weight that all heads share (`unit_norm`: no weight); with `freq` the first rot_dims numbers of every
 //                 head of q and k are turned by the token's position first (dimension i together with dimension
-//                 i + rot_dims / 2, angle position * freq[i]); q is then multiplied by 1 + coef * ln(floor((p + 1) / every) + 1) at
-//                 position p (every 0: no factor); all in 32-bit, rounded once, into the query rows and the cache slots.
+//                 i + rot_dims / 2, or `neighbours` 2i with 2i + 1, angle position * freq[i]), or with `norm_first` behind
+//                 the norm; q is then multiplied by 1 + coef * ln(floor((p + 1) / every) + 1) at position p (every 0: no
+//                 factor) and by a number per head (q_scale); all in 32-bit, rounded once, into the query rows and the
+//                 cache slots.  `v_from_k`: the values are the keys as projected, before norm and rotation.
 //   attend        one workgroup per new token, all heads.  Score heads s = h * maps + m (maps = 2: two score maps
 //                 per query head over the same values); s reads key head (h / (H / G)) * maps + m, values come from
 //                 value head h / (H / G).  A query at position i sees the key j <= i if
@@ -22,7 +24,8 @@
 //                 visible keys in 32-bit, normalised before anything else happens to it; with `sink` the denominator holds one more term exp(0); optionally the heads' weights
 //                 are mixed, w_h = sum_g talk[h, g] w_g; then the values.  maps = 2 ends with o = a_1 - lambda a_2;
 //                 head_norm divides a head's result by its root mean square (eps inside the root) and multiplies
-//                 by out_scale.  With gate products z (32-bit) the result is multiplied by sigmoid(z[n, h * dv + d]).
+//                 by out_scale.  With gate products z (32-bit) the result is multiplied by sigmoid(z[n, h * dv + d]), or with
+//                 gate_heads by sigmoid(z[n, h]).
 //
 // Keys are [pages, key heads, block, dk], values [pages, value heads, dv, block] (transposed inside a page).
 #include "common.h"
@@ -104,67 +107,264 @@ __global__ __launch_bounds__(AC_THREADS) void conv_state_kernel(
         ring[(size_t)(pos % (taps - 1)) * channels + c] = proj[(size_t)(first_row + pos - first_pos) * proj_stride + c];
 }
 
-// element d of a head after the rotation of its first rot_dims numbers (pairs i, i + rot_dims / 2)
-__device__ __forceinline__ float turned_element(const float* __restrict__ src, int d, int rot_dims, float position,
-                                                const float* __restrict__ freq) {
-    if (d >= rot_dims) return src[d];
-    const int h = rot_dims >> 1, i = d < h ? d : d - h;
-    const float2 sc = rotary_angle(position, freq[i]);  // (sine, cosine)
-    const float2 turned = rotate_pair(src[i], src[i + h], sc.y, sc.x);
-    return d < h ? turned.x : turned.y;
+// What norm_store is told.  Every head of q and k: turned by position and normed, in this order or the other.
+struct HeadStoreArgs {
+    int q_stride, proj_stride;
+    const float* proj;
+    const float* q_norm;  // [dk] weights, or null
+    const float* k_norm;
+    const float* q_scale;  // [q_heads]: the queries of a head are multiplied by a number of its own (null: 1)
+    const float* freq;     // [rot_dims / 2]
+    const float2* angles;  // [N, rot_dims / 2] (sine, cosine): given, it stands for freq
+    const int* positions;
+    const int* slots;
+    float eps, temp_coef;
+    int temp_every;
+    int n_tokens, q_heads, k_heads, dk, v_heads, dv, block_size, rot_dims;
+    int unit_norm;   // a norm without weights
+    int neighbours;  // dimensions 2i and 2i + 1 turn together (else i and i + rot_dims / 2)
+    int norm_first;  // the norm comes before the rotation
+    int v_from_k;    // values are the keys as projected (v_heads = k_heads, dv = dk; proj holds no values)
+};
+
+__device__ __forceinline__ float2 head_angle(const HeadStoreArgs& a, int n, float position, int i) {  // (sine, cosine)
+    return a.angles ? a.angles[(size_t)n * (a.rot_dims / 2) + i] : rotary_angle(position, a.freq[i]);
 }
 
-// grid: (tokens, query heads + key heads + value heads); one wave per head
+// number d of a head whose numbers are value(0) .. value(dk - 1), after the rotation
+template <class Value>
+__device__ __forceinline__ float turned_element(const HeadStoreArgs& a, Value value, int d, int n, float position) {
+    if (d >= a.rot_dims) return value(d);
+    const int h = a.rot_dims >> 1;
+    const int i = a.neighbours ? d >> 1 : (d < h ? d : d - h);
+    const int first = a.neighbours ? 2 * i : i, second = a.neighbours ? 2 * i + 1 : i + h;
+    const float2 sc = head_angle(a, n, position, i);
+    const float2 turned = rotate_pair(value(first), value(second), sc.y, sc.x);
+    return d == first ? turned.x : turned.y;
+}
+
+__device__ __forceinline__ float query_factor(const HeadStoreArgs& a, int n, int head) {
+    float factor = a.q_scale ? a.q_scale[head] : 1.f;
+    if (a.temp_every > 0) factor *= 1.f + a.temp_coef * logf((float)((a.positions[n] + 1) / a.temp_every + 1));
+    return factor;
+}
+
+// Any sizes.  grid: (tokens, query heads + key heads + value heads); one wave per head
 template <typename T>
-__global__ __launch_bounds__(LLMS_WAVE) void norm_store_kernel(
-    T* __restrict__ q_out, int q_stride, const float* __restrict__ proj, int proj_stride, const float* __restrict__ q_norm,
-    const float* __restrict__ k_norm, float eps, float temp_coef, int temp_every, const int* __restrict__ positions,
-    const int* __restrict__ slots, T* __restrict__ k_pool, T* __restrict__ v_pool, int q_heads, int k_heads, int dk,
-    int v_heads, int dv, int block_size, const float* __restrict__ freq, int rot_dims, int unit_norm) {
-    const int n = blockIdx.x, lane = threadIdx.x;
+__global__ __launch_bounds__(LLMS_WAVE) void norm_store_kernel(T* __restrict__ q_out, T* __restrict__ k_pool,
+                                                               T* __restrict__ v_pool, HeadStoreArgs a) {
+    const int n = blockIdx.x, lane = threadIdx.x, dk = a.dk, dv = a.dv;
     int head = blockIdx.y;
-    const float* row = proj + (size_t)n * proj_stride;
-    if (head < q_heads + k_heads) {
-        const bool is_q = head < q_heads;
+    const float* row = a.proj + (size_t)n * a.proj_stride;
+    if (head < a.q_heads + a.k_heads) {
+        const bool is_q = head < a.q_heads;
         const float* src = row + (size_t)head * dk;  // (keys follow the queries)
-        const float* w = is_q ? q_norm : k_norm;
+        const float* w = is_q ? a.q_norm : a.k_norm;
+        const bool normed = w || a.unit_norm;
+        const float position = a.rot_dims > 0 ? (float)a.positions[n] : 0.f;
+        auto raw = [&](int d) { return src[d]; };
         float mul = 1.f;
-        const float position = rot_dims > 0 ? (float)positions[n] : 0.f;
-        if (w || unit_norm) {
+        if (normed) {
             float ss = 0.f;
             for (int d = lane; d < dk; d += LLMS_WAVE) {
-                const float x = rot_dims > 0 ? turned_element(src, d, rot_dims, position, freq) : src[d];
+                const float x = a.norm_first ? src[d] : turned_element(a, raw, d, n, position);
                 ss = fmaf(x, x, ss);
             }
-            mul = 1.f / sqrtf(wave_sum(ss) / (float)dk + eps);
+            mul = 1.f / sqrtf(wave_sum(ss) / (float)dk + a.eps);
         }
-        float factor = 1.f;
-        if (is_q && temp_every > 0) factor = 1.f + temp_coef * logf((float)((positions[n] + 1) / temp_every + 1));
+        auto scaled = [&](float x, int d) { return w ? x * mul * w[d] : x * mul; };
+        auto normed_value = [&](int d) { return scaled(src[d], d); };
+        const float factor = is_q ? query_factor(a, n, head) : 1.f;
         T* dst;
         if (is_q) {
-            dst = q_out + (size_t)n * q_stride + (size_t)head * dk;
+            dst = q_out + (size_t)n * a.q_stride + (size_t)head * dk;
         } else {
-            if (!slots) return;
-            const int slot = slots[n];
+            if (!a.slots) return;
+            const int slot = a.slots[n];
             if (slot < 0) return;
-            const int page = slot / block_size, off = slot % block_size;
-            dst = k_pool + (((size_t)page * k_heads + (head - q_heads)) * block_size + off) * dk;
+            const int page = slot / a.block_size, off = slot % a.block_size;
+            dst = k_pool + (((size_t)page * a.k_heads + (head - a.q_heads)) * a.block_size + off) * dk;
         }
         for (int d = lane; d < dk; d += LLMS_WAVE) {
-            float x = (rot_dims > 0 ? turned_element(src, d, rot_dims, position, freq) : src[d]) * mul;
-            if (w) x *= w[d];
+            const float x = a.norm_first ? turned_element(a, normed_value, d, n, position)
+                                         : scaled(turned_element(a, raw, d, n, position), d);
             dst[d] = from_f32<T>(x * factor);
         }
         return;
     }
-    head -= q_heads + k_heads;
-    if (!slots) return;
-    const int slot = slots[n];
+    head -= a.q_heads + a.k_heads;
+    if (!a.slots) return;
+    const int slot = a.slots[n];
     if (slot < 0) return;
-    const int page = slot / block_size, off = slot % block_size;
-    const float* src = row + (size_t)(q_heads + k_heads) * dk + (size_t)head * dv;
+    const int page = slot / a.block_size, off = slot % a.block_size;
+    const float* src = a.v_from_k ? row + (size_t)(a.q_heads + head) * dk
+                                  : row + (size_t)(a.q_heads + a.k_heads) * dk + (size_t)head * dv;
     for (int d = lane; d < dv; d += LLMS_WAVE)
-        v_pool[(((size_t)page * v_heads + head) * dv + d) * block_size + off] = from_f32<T>(src[d]);
+        v_pool[(((size_t)page * a.v_heads + head) * dv + d) * a.block_size + off] = from_f32<T>(src[d]);
+}
+
+// Heads of up to 256 numbers, 4 to a lane: `lph` lanes (a power of two, at least dk / 4) hold a head of one token, so a
+// head's sum of squares is a few lane exchanges and a pair of the rotation lies in a lane (neighbours) or two.
+// The first `kv_blocks` workgroups take 16 tokens of one key or value head each: a page holds values transposed, so
+// they pass through LDS and leave with the tokens side by side in the lanes, which the memory system joins to whole
+// pieces where the tokens' slots follow one another.  The other workgroups take U heads of queries per group of lanes.
+#define HS_THREADS 256
+#define HS_TOKENS 16
+#define HS_MAX_DIM 256
+
+template <typename T>
+__device__ __forceinline__ void store4(T* dst, const float (&x)[4]) {
+    if constexpr (sizeof(T) == 2)
+        *reinterpret_cast<uint2*>(dst) = make_uint2(pack_bf16x2(x[0], x[1]), pack_bf16x2(x[2], x[3]));
+    else
+        *reinterpret_cast<float4*>(dst) = make_float4(x[0], x[1], x[2], x[3]);
+}
+
+// x: the lane's 4 numbers (4 li ..) of a head of token n
+__device__ __forceinline__ void turn4(const HeadStoreArgs& a, float (&x)[4], int li, int n, bool live) {
+    const int half = a.rot_dims >> 1;
+    const float2* row = a.angles + (size_t)n * half;
+    if (a.neighbours) {
+#pragma unroll
+        for (int p = 0; p < 2; ++p) {
+            const int i = 2 * li + p;
+            if (live && i < half) {
+                const float2 sc = row[i];
+                const float2 t = rotate_pair(x[2 * p], x[2 * p + 1], sc.y, sc.x);
+                x[2 * p] = t.x, x[2 * p + 1] = t.y;
+            }
+        }
+        return;
+    }
+    const int hl = half >> 2;  // lanes that hold the first partners (half is a multiple of 4 here)
+    const bool turns = li < 2 * hl, low = li < hl;
+    const int lane = threadIdx.x % LLMS_WAVE, partner = turns ? (low ? lane + hl : lane - hl) : lane;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+        const float other = __shfl(x[e], partner, LLMS_WAVE);
+        if (live && turns) {
+            const float2 sc = row[4 * (low ? li : li - hl) + e];
+            const float2 t = low ? rotate_pair(x[e], other, sc.y, sc.x) : rotate_pair(other, x[e], sc.y, sc.x);
+            x[e] = low ? t.x : t.y;
+        }
+    }
+}
+
+__device__ __forceinline__ void prepare4(const HeadStoreArgs& a, float (&x)[4], const float* __restrict__ w, int li, int lph,
+                                         int n, bool live) {
+    if (a.rot_dims > 0 && !a.norm_first) turn4(a, x, li, n, live);
+    if (w || a.unit_norm) {
+        float ss = 0.f;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss = fmaf(x[e], x[e], ss);
+        for (int o = lph >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, LLMS_WAVE);
+        const float mul = 1.f / sqrtf(ss / (float)a.dk + a.eps);
+        float4 wv = make_float4(1.f, 1.f, 1.f, 1.f);
+        if (w && 4 * li < a.dk) wv = *reinterpret_cast<const float4*>(w + 4 * li);
+        x[0] = x[0] * mul * wv.x, x[1] = x[1] * mul * wv.y, x[2] = x[2] * mul * wv.z, x[3] = x[3] * mul * wv.w;
+    }
+    if (a.rot_dims > 0 && a.norm_first) turn4(a, x, li, n, live);
+}
+
+template <typename T, int U>
+__global__ __launch_bounds__(HS_THREADS) void head_store_kernel(T* __restrict__ q_out, T* __restrict__ k_pool,
+                                                                T* __restrict__ v_pool, HeadStoreArgs a, int lph, int kv_blocks) {
+    __shared__ float tile[HS_TOKENS * (HS_MAX_DIM + 1)];
+    __shared__ long long place[HS_TOKENS];  // of number 0 of the token's value (-1: none)
+    const int tid = threadIdx.x, li = tid & (lph - 1), group = tid / lph, groups = HS_THREADS / lph;
+    const int dk = a.dk, dv = a.dv;
+    const bool in_head = 4 * li < dk;
+    if ((int)blockIdx.x >= kv_blocks) {
+        const int first = ((int)blockIdx.x - kv_blocks) * groups * U + group, total = a.n_tokens * a.q_heads;
+        float x[U][4];
+        int tok[U], head[U];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const int item = min(first + u * groups, total - 1);
+            tok[u] = item / a.q_heads, head[u] = item - tok[u] * a.q_heads;
+            float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (in_head) v = *reinterpret_cast<const float4*>(a.proj + (size_t)tok[u] * a.proj_stride + (size_t)head[u] * dk + 4 * li);
+            x[u][0] = v.x, x[u][1] = v.y, x[u][2] = v.z, x[u][3] = v.w;
+        }
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            prepare4(a, x[u], a.q_norm, li, lph, tok[u], in_head);
+            const float factor = query_factor(a, tok[u], head[u]);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) x[u][e] *= factor;
+            if (in_head && first + u * groups < total)
+                store4<T>(q_out + (size_t)tok[u] * a.q_stride + (size_t)head[u] * dk + 4 * li, x[u]);
+        }
+        return;
+    }
+    const int roles = a.k_heads + (a.v_from_k ? 0 : a.v_heads);
+    const int n0 = ((int)blockIdx.x / roles) * HS_TOKENS, role = (int)blockIdx.x % roles;
+    const bool is_k = role < a.k_heads;
+    const int v_head = is_k ? role : role - a.k_heads;
+    if (tid < HS_TOKENS) {
+        const int slot = n0 + tid < a.n_tokens ? a.slots[n0 + tid] : -1;
+        const int page = slot / a.block_size, off = slot - page * a.block_size;
+        place[tid] = slot < 0 ? -1 : ((long long)page * a.v_heads + v_head) * dv * a.block_size + off;
+    }
+    const int pitch = dv + 1;
+    if (is_k) {
+        for (int t0 = 0; t0 < HS_TOKENS; t0 += groups) {
+            const int t = t0 + group, n = min(n0 + t, a.n_tokens - 1);
+            const bool live = t < HS_TOKENS && n0 + t < a.n_tokens;
+            const int slot = live ? a.slots[n] : -1;
+            float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (in_head) v = *reinterpret_cast<const float4*>(a.proj + (size_t)n * a.proj_stride + (size_t)(a.q_heads + role) * dk + 4 * li);
+            float x[4] = {v.x, v.y, v.z, v.w};
+            if (a.v_from_k && live && in_head) {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) tile[t * pitch + 4 * li + e] = x[e];
+            }
+            prepare4(a, x, a.k_norm, li, lph, n, in_head);
+            if (in_head && slot >= 0) {
+                const int page = slot / a.block_size, off = slot - page * a.block_size;
+                store4<T>(k_pool + (((size_t)page * a.k_heads + role) * a.block_size + off) * dk + 4 * li, x);
+            }
+        }
+        if (!a.v_from_k) return;
+    } else {
+        const float* src = a.proj + (size_t)(a.q_heads + a.k_heads) * dk + (size_t)v_head * dv;
+        for (int i = tid; i < HS_TOKENS * dv; i += HS_THREADS) {
+            const int t = i / dv, d = i - t * dv;
+            if (n0 + t < a.n_tokens) tile[t * pitch + d] = src[(size_t)(n0 + t) * a.proj_stride + d];
+        }
+    }
+    __syncthreads();
+    for (int i = tid; i < HS_TOKENS * dv; i += HS_THREADS) {
+        const int t = i % HS_TOKENS, d = i / HS_TOKENS;
+        const long long at = place[t];
+        if (at >= 0) v_pool[at + (long long)d * a.block_size] = from_f32<T>(tile[t * pitch + d]);
+    }
+}
+
+template <typename T>
+static int launch_norm_store(T* q_out, T* k_pool, T* v_pool, const HeadStoreArgs& a, hipStream_t stream) {
+    const int half = a.rot_dims / 2;
+    const bool four = a.dk % 4 == 0 && a.dk <= HS_MAX_DIM && a.dv <= HS_MAX_DIM && a.proj_stride % 4 == 0 && a.q_stride % 4 == 0 &&
+                      ((uintptr_t)a.proj % 16) == 0 && ((uintptr_t)q_out % 16) == 0 && (!k_pool || ((uintptr_t)k_pool % 16) == 0) &&
+                      ((uintptr_t)a.q_norm % 16) == 0 && ((uintptr_t)a.k_norm % 16) == 0 &&
+                      (a.rot_dims == 0 || (a.angles && (a.neighbours || half % 4 == 0)));
+    if (four) {
+        int lph = 1;
+        while (4 * lph < a.dk) lph *= 2;
+        const int groups = HS_THREADS / lph;
+        const long long items = (long long)a.n_tokens * a.q_heads;
+        const long long kv_blocks = a.slots ? (long long)((a.n_tokens + HS_TOKENS - 1) / HS_TOKENS) * (a.k_heads + (a.v_from_k ? 0 : a.v_heads)) : 0;
+        const int per = items >= 4096 ? 4 : 1;
+        const long long q_blocks = (items + (long long)groups * per - 1) / (groups * per);
+        LLMS_REQUIRE(items < (1ll << 30) && kv_blocks + q_blocks < (1ll << 31), "norm_store: too many tokens for one launch");
+        const unsigned grid = (unsigned)(kv_blocks + q_blocks);
+        if (per == 4) head_store_kernel<T, 4><<<grid, HS_THREADS, 0, stream>>>(q_out, k_pool, v_pool, a, lph, (int)kv_blocks);
+        else head_store_kernel<T, 1><<<grid, HS_THREADS, 0, stream>>>(q_out, k_pool, v_pool, a, lph, (int)kv_blocks);
+    } else {
+        dim3 grid(a.n_tokens, a.q_heads + a.k_heads + a.v_heads);
+        norm_store_kernel<T><<<grid, LLMS_WAVE, 0, stream>>>(q_out, k_pool, v_pool, a);
+    }
+    LLMS_LAUNCH_CHECK();
 }
 
 // ------------------------------------------------------------------------------------------- attention
@@ -178,6 +378,7 @@ struct ComposedArgs {
     int dist_reach;
     const float* gate;  // 32-bit products [N, gate_stride], or null
     int gate_stride;
+    int gate_heads;  // the gate is one number per head, gate[n, h], instead of one per element
     int sink;  // the softmax's denominator holds one more term, exp(0): a key of score zero that has no value
 };
 
@@ -353,7 +554,7 @@ __global__ __launch_bounds__(AC_THREADS) void attend_composed_kernel(
             float o = acc_o[(h * a.maps) * dv + d];
             if (a.maps == 2) o -= a.lambda * acc_o[(h * 2 + 1) * dv + d];
             o *= mul;
-            if (a.gate) o /= 1.f + expf(-a.gate[(size_t)n * a.gate_stride + h * dv + d]);
+            if (a.gate) o /= 1.f + expf(-a.gate[(size_t)n * a.gate_stride + (a.gate_heads ? h : h * dv + d)]);
             orow[h * dv + d] = from_f32<T>(o);
         }
     }
@@ -399,27 +600,26 @@ int llms_conv_store(int dtype, void* q_out, int q_stride, const float* proj, int
 int llms_norm_store(int dtype, void* q_out, int q_stride, const float* proj, int proj_stride, const float* q_norm,
                     const float* k_norm, float eps, float temp_coef, int temp_every, const int* positions, const int* slots,
                     void* k_pool, void* v_pool, int n_tokens, int q_heads, int k_heads, int dk, int v_heads, int dv,
-                    int block_size, const float* freq, int rot_dims, int unit_norm, hipStream_t stream) {
+                    int block_size, const float* freq, const float* angles, int rot_dims, int unit_norm, int neighbours,
+                    int norm_first, const float* q_scale, int v_from_k, hipStream_t stream) {
     LLMS_REQUIRE(n_tokens > 0 && q_heads > 0 && k_heads >= 0 && v_heads >= 0 && dk > 0 && dv > 0, "norm_store: sizes must be positive");
-    LLMS_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= dk && (rot_dims == 0 || (freq && positions)),
-                 "norm_store: an even number of turned dimensions within a head, with frequencies and positions");
+    LLMS_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= dk && (rot_dims == 0 || angles || (freq && positions)),
+                 "norm_store: an even number of turned dimensions within a head, with angles or frequencies and positions");
+    LLMS_REQUIRE(((uintptr_t)angles % 8) == 0, "norm_store: the table of angles must be 8-byte aligned");
     LLMS_REQUIRE(temp_every == 0 || positions, "norm_store: a factor by position needs the positions");
     LLMS_REQUIRE(!slots || (k_pool && v_pool && block_size > 0), "norm_store: slots given without pools");
     LLMS_REQUIRE(q_heads + k_heads + v_heads <= 65535, "norm_store: up to 65,535 heads in all");
-    dim3 grid(n_tokens, q_heads + k_heads + v_heads);
-    if (dtype == 0)
-        norm_store_kernel<float><<<grid, LLMS_WAVE, 0, stream>>>((float*)q_out, q_stride, proj, proj_stride, q_norm, k_norm, eps,
-                                                                 temp_coef, temp_every, positions, slots, (float*)k_pool,
-                                                                 (float*)v_pool, q_heads, k_heads, dk, v_heads, dv, block_size,
-                                                                 freq, rot_dims, unit_norm);
-    else if (dtype == 1)
-        norm_store_kernel<bf16><<<grid, LLMS_WAVE, 0, stream>>>((bf16*)q_out, q_stride, proj, proj_stride, q_norm, k_norm, eps,
-                                                                temp_coef, temp_every, positions, slots, (bf16*)k_pool,
-                                                                (bf16*)v_pool, q_heads, k_heads, dk, v_heads, dv, block_size,
-                                                                freq, rot_dims, unit_norm);
-    else
-        LLMS_REQUIRE(false, "norm_store: dtype must be 0 (float32) or 1 (bfloat16)");
-    LLMS_LAUNCH_CHECK();
+    LLMS_REQUIRE(!v_from_k || (v_heads == k_heads && dv == dk), "norm_store: values that are the keys have their heads and size");
+    HeadStoreArgs a;
+    a.q_stride = q_stride, a.proj_stride = proj_stride, a.proj = proj, a.q_norm = q_norm, a.k_norm = k_norm, a.q_scale = q_scale;
+    a.freq = freq, a.angles = reinterpret_cast<const float2*>(angles), a.positions = positions, a.slots = slots;
+    a.eps = eps, a.temp_coef = temp_coef, a.temp_every = temp_every;
+    a.n_tokens = n_tokens, a.q_heads = q_heads, a.k_heads = k_heads, a.dk = dk, a.v_heads = v_heads, a.dv = dv;
+    a.block_size = block_size > 0 ? block_size : 1, a.rot_dims = rot_dims;
+    a.unit_norm = unit_norm, a.neighbours = neighbours, a.norm_first = norm_first, a.v_from_k = v_from_k;
+    if (dtype == 0) return launch_norm_store<float>((float*)q_out, (float*)k_pool, (float*)v_pool, a, stream);
+    if (dtype == 1) return launch_norm_store<bf16>((bf16*)q_out, (bf16*)k_pool, (bf16*)v_pool, a, stream);
+    LLMS_REQUIRE(false, "norm_store: dtype must be 0 (float32) or 1 (bfloat16)");
 }
 
 int llms_conv_state(float* state, size_t state_slot_stride, const int* state_slots, const float* proj, int proj_stride,
@@ -438,7 +638,7 @@ int llms_attend_composed(int dtype, void* out, int out_stride, const void* q, in
                          int kv_heads, int maps,
                          int dk, int dv, int block_size, int window, int keep_first, int chunk, float scale,
                          const float* slopes, const float* talk, float lambda, int head_norm, float eps, float out_scale,
-                         const float* dist_bias, int dist_reach, const float* gate, int gate_stride, int sink,
+                         const float* dist_bias, int dist_reach, const float* gate, int gate_stride, int gate_heads, int sink,
                          hipStream_t stream) {
     LLMS_REQUIRE(n_tokens > 0 && heads > 0 && kv_heads > 0 && dk > 0 && dv > 0, "attend_composed: sizes must be positive");
     LLMS_REQUIRE(!dist_bias || dist_reach >= 0, "attend_composed: a distance table has at least one entry per head");
@@ -454,7 +654,7 @@ int llms_attend_composed(int dtype, void* out, int out_stride, const void* q, in
     a.heads = heads, a.kv_heads = kv_heads, a.maps = maps, a.dk = dk, a.dv = dv, a.block_size = block_size;
     a.window = window, a.keep_first = keep_first, a.chunk = chunk;
     a.scale = scale, a.lambda = lambda, a.eps = eps, a.out_scale = out_scale, a.head_norm = head_norm;
-    a.dist_bias = dist_bias, a.dist_reach = dist_reach, a.gate = gate, a.gate_stride = gate_stride, a.sink = sink;
+    a.dist_bias = dist_bias, a.dist_reach = dist_reach, a.gate = gate, a.gate_stride = gate_stride, a.gate_heads = gate_heads, a.sink = sink;
     if (dtype == 0) {
         auto kernel = attend_composed_kernel<float>;
         if (lds > 48 * 1024)

@@ -53,6 +53,7 @@ struct MfmaArgs {
     const float* dist_bias;  // [heads, dist_reach + 1]: a bias per head and distance, the last entry for everything beyond; or null
     const float* gate;       // 32-bit products [N, gate_stride]: the result is multiplied by their sigmoid; or null
     int dist_reach, gate_stride;
+    int gate_heads;  // one number per head, gate[n, h], instead of one per element
     int out_stride, q_stride, max_blocks;
     int seq_begin, n_seqs, blocks_per_seq;
     int heads, kv_heads, grp, dk, dv, block_size;
@@ -598,12 +599,13 @@ __global__ __launch_bounds__(THREADS) void attend_mfma_kernel(const MfmaArgs a) 
             continue;
         }
         bf16* orow = a.out + (size_t)(row0 + t0 + u_tl[uu]) * a.out_stride + (size_t)u_h[uu] * dv + 4 * q4;
-        const float* grow = a.gate ? a.gate + (size_t)(row0 + t0 + u_tl[uu]) * a.gate_stride + (size_t)u_h[uu] * dv + 4 * q4 : nullptr;
+        const float* grow = a.gate ? a.gate + (size_t)(row0 + t0 + u_tl[uu]) * a.gate_stride + (a.gate_heads ? (size_t)u_h[uu] : (size_t)u_h[uu] * dv + 4 * q4) : nullptr;
+        if (grow && a.gate_heads) norm /= 1.f + expf(-grow[0]);
 #pragma unroll
         for (int t = 0; t < MAXTV; ++t)
             if (t < dvt) {
                 f32x4 o = acc_o[uu][0][t] * norm;
-                if (grow) {
+                if (grow && !a.gate_heads) {
                     const f32x4 z = *reinterpret_cast<const f32x4*>(grow + 16 * t);
 #pragma unroll
                     for (int r = 0; r < 4; ++r) o[r] /= 1.f + expf(-z[r]);
@@ -675,7 +677,7 @@ int llms_attend_composed_mfma(void* out, int out_stride, const void* q, int q_st
                               int heads, int kv_heads, int maps, int dk, int dv, int block_size, int window,
                               int keep_first, int chunk, float scale, const float* slopes, const float* talk, float lambda,
                               int head_norm, float eps, float out_scale, int shares, float* ws_stats, float* ws_o, int ws_rows,
-                              const float* dist_bias, int dist_reach, const float* gate, int gate_stride, int sink,
+                              const float* dist_bias, int dist_reach, const float* gate, int gate_stride, int gate_heads, int sink,
                               hipStream_t stream) {
     LLMS_REQUIRE(n_seqs > 0 && max_new > 0 && heads > 0 && kv_heads > 0, "attend_composed_mfma: sizes must be positive");
     LLMS_REQUIRE(!(sink && talk), "attend_composed_mfma: no sink where heads are mixed");
@@ -692,8 +694,8 @@ int llms_attend_composed_mfma(void* out, int out_stride, const void* q, int q_st
     a.block_tables = block_tables, a.table_rows = table_rows, a.cu_seqlens = cu_seqlens, a.context_lens = context_lens;
     a.slopes = slopes, a.talk = talk;
     LLMS_REQUIRE(!dist_bias || dist_reach >= 0, "attend_composed_mfma: a distance table has at least one entry per head");
-    LLMS_REQUIRE(!gate || (!talk && gate_stride % 4 == 0), "attend_composed_mfma: gate rows are 16-byte aligned, and no gate where heads are mixed");
-    a.dist_bias = dist_bias, a.dist_reach = dist_reach, a.gate = gate, a.gate_stride = gate_stride;
+    LLMS_REQUIRE(!gate || (!talk && (gate_heads || gate_stride % 4 == 0)), "attend_composed_mfma: gate rows are 16-byte aligned, and no gate where heads are mixed");
+    a.dist_bias = dist_bias, a.dist_reach = dist_reach, a.gate = gate, a.gate_stride = gate_stride, a.gate_heads = gate_heads;
     a.out_stride = out_stride, a.q_stride = q_stride, a.max_blocks = max_blocks, a.seq_begin = seq_begin, a.n_seqs = n_seqs;
     a.heads = heads, a.kv_heads = kv_heads, a.grp = heads / kv_heads, a.dk = dk, a.dv = dv, a.block_size = block_size;
     a.window = window, a.keep_first = keep_first, a.chunk = chunk;

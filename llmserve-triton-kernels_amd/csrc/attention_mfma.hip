@@ -54,6 +54,24 @@ __device__ __forceinline__ uint4 keep_elements(uint4 v, int first, int last) {
     return make_uint4(w[0], w[1], w[2], w[3]);
 }
 
+// In the library built with head gates (attention_gated.hip) `gate` holds one 32-bit number per token and head,
+// gate[row * gate_stride + head], and a head's result is multiplied by its sigmoid where it is divided by the sum of its
+// weights, in every kernel that finishes a column.
+#ifdef LLMS_ATTENTION_HEAD_GATED
+constexpr bool HEAD_GATE = true;
+#else
+constexpr bool HEAD_GATE = false;
+#endif
+#if !defined(LLMS_ATTENTION_BIASED) && !defined(LLMS_ATTENTION_HEAD_GATED)
+#define LLMS_ATTENTION_PLAIN 1
+#endif
+
+// What a column's sum is multiplied by at the end: 1 / l, times sigmoid(z) where heads are gated.
+__device__ __forceinline__ float column_factor(float l, float z) {
+    if constexpr (HEAD_GATE) return 1.f / (l * (1.f + expf(-z)));
+    return 1.f / l;
+}
+
 struct AttnArgs {
     bf16* out;
     int out_stride;
@@ -87,7 +105,7 @@ struct AttnArgs {
     int one_token_from;
     // prompts only: a bias per head and distance, [heads, dist_reach + 1] with the last entry for everything beyond,
     // added to the scaled score (null: none), and 32-bit products [rows, gate_stride] by whose sigmoid the result is
-    // multiplied (null: none)
+    // multiplied (null: none; with head gates: one number per head, prompts and decoding)
     const float* dist_bias;
     int dist_reach;
     const float* gate;
@@ -275,7 +293,7 @@ __device__ __forceinline__ float2 load_across(const float* p) {
 // is used (a split beyond the last is the last once more, with weight 0).
 template <int DB, int SMAX>
 __device__ __forceinline__ void merge_shares(const AttnArgs& a, size_t item0, bool col_ok, int wave, int nw, int g,
-                                             bf16* orow) {
+                                             bf16* orow, float gate_z) {
     constexpr int D = DB * 16;
     if (!col_ok) return;
     const int S = a.num_splits;
@@ -291,7 +309,7 @@ __device__ __forceinline__ void merge_shares(const AttnArgs& a, size_t item0, bo
         w[s] = (s < S && ml[s].x != -INFINITY) ? exp2_fast(ml[s].x - m_tot) : 0.f;
         if (s < S && ml[s].x != -INFINITY) l_tot += ml[s].y * w[s];
     }
-    const float inv = 1.f / l_tot;
+    const float inv = column_factor(l_tot, gate_z);
     for (int m = wave; m < DB; m += nw) {
         float2 lo[SMAX], hi[SMAX];
 #pragma unroll
@@ -360,6 +378,8 @@ __global__ __launch_bounds__(NW* LLMS_WAVE) void attn_mfma_kernel(const AttnArgs
                     ? *reinterpret_cast<const uint4*>(a.q + (size_t)(tok0 + c_tok) * a.q_stride + (size_t)head * D + d)
                     : zero;
     }
+    float gate_z = 0.f;  // (asked for with the queries: at the end it would be a trip to memory of its own)
+    if constexpr (HEAD_GATE) gate_z = col_ok ? a.gate[(size_t)(tok0 + c_tok) * a.gate_stride + head] : 0.f;
     if (t_first >= n_new || ctx <= 0) return;  // (uniform over the workgroup)
 
     const int p_col = col_ok ? ctx - n_new + c_tok : -1;  // absolute position of the column's token
@@ -521,7 +541,7 @@ __global__ __launch_bounds__(NW* LLMS_WAVE) void attn_mfma_kernel(const AttnArgs
         }
         if (!col_ok) continue;
         if (a.num_splits == 1) {
-            const float inv = 1.f / l_tot;
+            const float inv = column_factor(l_tot, gate_z);
             uint2 pk;
             pk.x = pack_bf16(o.x * inv, o.y * inv);
             pk.y = pack_bf16(o.z * inv, o.w * inv);
@@ -557,10 +577,10 @@ __global__ __launch_bounds__(NW* LLMS_WAVE) void attn_mfma_kernel(const AttnArgs
         if (!is_last) return;
         const size_t item0 = ((size_t)(tok0 + c_tok) * a.n_heads + head) * a.num_splits;
         bf16* orow = a.out + (size_t)(tok0 + c_tok) * a.out_stride + (size_t)head * D;
-        if (a.num_splits <= 2) merge_shares<DB, 2>(a, item0, col_ok, wave, nw, g, orow);
-        else if (a.num_splits <= 4) merge_shares<DB, 4>(a, item0, col_ok, wave, nw, g, orow);
-        else if (a.num_splits <= 8) merge_shares<DB, 8>(a, item0, col_ok, wave, nw, g, orow);
-        else merge_shares<DB, 16>(a, item0, col_ok, wave, nw, g, orow);
+        if (a.num_splits <= 2) merge_shares<DB, 2>(a, item0, col_ok, wave, nw, g, orow, gate_z);
+        else if (a.num_splits <= 4) merge_shares<DB, 4>(a, item0, col_ok, wave, nw, g, orow, gate_z);
+        else if (a.num_splits <= 8) merge_shares<DB, 8>(a, item0, col_ok, wave, nw, g, orow, gate_z);
+        else merge_shares<DB, 16>(a, item0, col_ok, wave, nw, g, orow, gate_z);
     }
 }
 
@@ -864,7 +884,9 @@ __global__ __launch_bounds__((TWIN ? 2 : 1) * WB * LLMS_WAVE, (TWIN && DB <= 4) 
             }
             continue;
         }
-        const float inv = 1.f / l_run[cg];
+        float gate_z = 0.f;
+        if constexpr (HEAD_GATE) gate_z = a.gate[(size_t)(tok0 + c_tok[cg]) * a.gate_stride + head];
+        const float inv = column_factor(l_run[cg], gate_z);
         bf16* orow = a.out + (size_t)(tok0 + c_tok[cg]) * a.out_stride + (size_t)head * D;
         if (BIAS && a.gate) {
             const float* grow = a.gate + (size_t)(tok0 + c_tok[cg]) * a.gate_stride + (size_t)head * D;
@@ -892,7 +914,8 @@ __global__ __launch_bounds__((TWIN ? 2 : 1) * WB * LLMS_WAVE, (TWIN && DB <= 4) 
 // token, blockIdx.y: which blockDim.x of the token's heads * head_dim / 4 pieces).
 __global__ __launch_bounds__(256) void attn_merge_kernel(bf16* __restrict__ out, int out_stride, const float* __restrict__ ws_o,
                                                          const float* __restrict__ ws_ml, int token_begin, int n_heads,
-                                                         int head_dim, int num_splits) {
+                                                         int head_dim, int num_splits, const float* __restrict__ gate,
+                                                         int gate_stride) {
     const int token = token_begin + blockIdx.x;
     const int q4 = head_dim / 4;
     const int idx = blockIdx.y * blockDim.x + threadIdx.x;
@@ -918,7 +941,9 @@ __global__ __launch_bounds__(256) void attn_merge_kernel(bf16* __restrict__ out,
                 o.w += p.w * w;
             }
         }
-        const float inv = 1.f / l_tot;
+        float gate_z = 0.f;
+        if constexpr (HEAD_GATE) gate_z = gate[(size_t)token * gate_stride + head];
+        const float inv = column_factor(l_tot, gate_z);
         uint2 pk;
         pk.x = pack_bf16(o.x * inv, o.y * inv);
         pk.y = pack_bf16(o.z * inv, o.w * inv);
@@ -948,10 +973,10 @@ static void launch_prompt_cg(dim3 grid, bool twin, const AttnArgs& a, hipStream_
 
 // Few tokens (decoding): small workgroups, so that the merge reaches many CUs; many tokens: 256 threads each.
 static void launch_merge(void* out, int out_stride, const float* ws_o, const float* ws_ml, int token_begin, int n_tokens,
-                         int n_heads, int head_dim, int num_splits, hipStream_t stream) {
+                         int n_heads, int head_dim, int num_splits, const float* gate, int gate_stride, hipStream_t stream) {
     const int threads = n_tokens <= 64 ? 64 : 256, pieces = n_heads * (head_dim / 4);
     attn_merge_kernel<<<dim3(n_tokens, (pieces + threads - 1) / threads), threads, 0, stream>>>(
-        (bf16*)out, out_stride, ws_o, ws_ml, token_begin, n_heads, head_dim, num_splits);
+        (bf16*)out, out_stride, ws_o, ws_ml, token_begin, n_heads, head_dim, num_splits, gate, gate_stride);
 }
 
 #ifdef LLMS_ATTENTION_BIASED
@@ -1086,7 +1111,7 @@ static int attention_mfma_launch(void* out, int out_stride, const void* q, int q
                 fprintf(stderr, "llmserve kernel launch failed: %s\n", hipGetErrorString(e1));
                 return LLMS_ERR_LAUNCH;
             }
-            launch_merge(out, out_stride, ws_o, ws_ml, token_begin, n_tokens, n_heads, head_dim, num_splits, stream);
+            launch_merge(out, out_stride, ws_o, ws_ml, token_begin, n_tokens, n_heads, head_dim, num_splits, gate, gate_stride, stream);
         }
     } else {
         // twins (8 waves, two tiles a round) where a workgroup per CU is left that way; wider heads would not fit
@@ -1120,13 +1145,13 @@ static int attention_mfma_launch(void* out, int out_stride, const void* q, int q
                 fprintf(stderr, "llmserve kernel launch failed: %s\n", hipGetErrorString(e1));
                 return LLMS_ERR_LAUNCH;
             }
-            launch_merge(out, out_stride, ws_o, ws_ml, token_begin, n_tokens, n_heads, head_dim, num_splits, stream);
+            launch_merge(out, out_stride, ws_o, ws_ml, token_begin, n_tokens, n_heads, head_dim, num_splits, gate, gate_stride, stream);
         }
     }
     LLMS_LAUNCH_CHECK();
 }
 
-#ifndef LLMS_ATTENTION_BIASED
+#ifdef LLMS_ATTENTION_PLAIN
 // The plain attention: no distance table, no gate.
 int llms_attention_mfma(void* out, int out_stride, const void* q, int q_stride, const void* k_pool,
                         const void* v_pool, const int* block_tables, const int* table_rows, int max_blocks,
@@ -1139,6 +1164,21 @@ int llms_attention_mfma(void* out, int out_stride, const void* q, int q_stride, 
                                  context_lens, seq_begin, n_seqs, max_new, token_begin, n_tokens, n_heads, n_kv_heads, head_dim,
                                  block_size, window, scale, split_waves, num_splits, waves, ws_o, ws_ml, arrive, n_arrive,
                                  nullptr, 0, nullptr, 0, stream);
+}
+#elif defined(LLMS_ATTENTION_HEAD_GATED)
+// The plain attention with every head's result multiplied by the sigmoid of one 32-bit number per token and head,
+// gate[row * gate_stride + head].
+int llms_attention_mfma_gated(void* out, int out_stride, const void* q, int q_stride, const void* k_pool,
+                              const void* v_pool, const int* block_tables, const int* table_rows, int max_blocks,
+                              const int* cu_seqlens, const int* context_lens, int seq_begin, int n_seqs, int max_new,
+                              int token_begin, int n_tokens, int n_heads, int n_kv_heads, int head_dim, int block_size,
+                              int window, float scale, int split_waves, int num_splits, int waves, float* ws_o, float* ws_ml,
+                              unsigned* arrive, int n_arrive, const float* gate, int gate_stride, hipStream_t stream) {
+    LLMS_REQUIRE(gate && gate_stride >= n_heads, "attention_mfma_gated: a gate row has a number per head");
+    return attention_mfma_launch(out, out_stride, q, q_stride, k_pool, v_pool, block_tables, table_rows, max_blocks, cu_seqlens,
+                                 context_lens, seq_begin, n_seqs, max_new, token_begin, n_tokens, n_heads, n_kv_heads, head_dim,
+                                 block_size, window, scale, split_waves, num_splits, waves, ws_o, ws_ml, arrive, n_arrive,
+                                 nullptr, 0, gate, gate_stride, stream);
 }
 #else
 // Prompt portions with a bias per head and distance on the scaled scores (dist_bias float [n_heads, dist_reach + 1],
@@ -1163,7 +1203,7 @@ int llms_attention_prompt_biased(void* out, int out_stride, const void* q, int q
 
 }  // extern "C"
 
-#ifndef LLMS_ATTENTION_BIASED
+#ifdef LLMS_ATTENTION_PLAIN
 
 // ---------------------------------------------------------------------------------------------------------
 // Decoding with the keys of a request shared out to several workgroups, without a workspace from the caller:
@@ -1227,4 +1267,4 @@ int llms_attention_decode_noalloc(void* out, int out_stride, const void* q, int 
 }
 
 }  // extern "C"
-#endif  // LLMS_ATTENTION_BIASED
+#endif  // LLMS_ATTENTION_PLAIN

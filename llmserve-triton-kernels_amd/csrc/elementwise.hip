@@ -388,8 +388,14 @@ __global__ __launch_bounds__(256) void rope_store_bf16_vec_kernel(bf16* __restri
 // ------------------------------------------------------------------ SiLU(gate) * up
 // gate_up row = [gate (inter) | up (inter)]; out = T(T(silu(gate)) * up), the reference's
 // rounding points (src/llmserve/model/llama.py:120).
-template <typename T>
-__global__ void silu_mul_kernel(T* __restrict__ out, const T* __restrict__ gate_up, int inter, size_t total) {
+// CLAMPED: g sigmoid(1.702 g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit), in 32-bit, rounded once.
+__device__ __forceinline__ float clamped_unit(float gate, float up, float limit) {
+    const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+    return g / (1.f + expf(-1.702f * g)) * (u + 1.f);
+}
+
+template <typename T, bool CLAMPED>
+__global__ void silu_mul_kernel(T* __restrict__ out, const T* __restrict__ gate_up, int inter, size_t total, float limit) {
     const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= total) return;
     const size_t n = idx / inter;
@@ -397,13 +403,18 @@ __global__ void silu_mul_kernel(T* __restrict__ out, const T* __restrict__ gate_
     const T* row = gate_up + n * 2 * (size_t)inter;
     const float g = to_f32(row[i]);
     const float u = to_f32(row[inter + i]);
+    if constexpr (CLAMPED) {
+        out[idx] = from_f32<T>(clamped_unit(g, u, limit));
+        return;
+    }
     const float s = round_to<T>(g / (1.f + expf(-g)));
     out[idx] = from_f32<T>(s * u);
 }
 
 // bfloat16 rows of inter % 8 == 0: 8 elements per thread, 16-byte loads and stores.
+template <bool CLAMPED>
 __global__ void silu_mul_bf16_vec_kernel(bf16* __restrict__ out, const bf16* __restrict__ gate_up, int inter,
-                                         size_t total_chunks) {
+                                         size_t total_chunks, float limit) {
     const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= total_chunks) return;
     const int cpr = inter / 8;  // chunks per row
@@ -420,11 +431,40 @@ __global__ void silu_mul_bf16_vec_kernel(bf16* __restrict__ out, const bf16* __r
         for (int h = 0; h < 2; ++h) {
             const float g = bf16_bits_to_f32((uint16_t)(h ? gw[j] >> 16 : gw[j] & 0xffffu));
             const float u = bf16_bits_to_f32((uint16_t)(h ? uw[j] >> 16 : uw[j] & 0xffffu));
-            r2[h] = round_to<bf16>(g / (1.f + expf(-g))) * u;
+            r2[h] = CLAMPED ? clamped_unit(g, u, limit) : round_to<bf16>(g / (1.f + expf(-g))) * u;
         }
         ow[j] = pack_bf16x2(r2[0], r2[1]);
     }
     reinterpret_cast<uint4*>(out)[idx] = make_uint4(ow[0], ow[1], ow[2], ow[3]);
+}
+
+// ------------------------------------------------------------------ max(x, 0)^2 in place
+// 16 bytes a thread; the last thread takes what is left of the array.
+template <typename T>
+__global__ void squared_relu_kernel(T* __restrict__ x, size_t n) {
+    constexpr int PER = 16 / sizeof(T);
+    const size_t i = ((size_t)blockIdx.x * blockDim.x + threadIdx.x) * PER;
+    if (i >= n) return;
+    if (i + PER <= n) {
+        const uint4 raw = *reinterpret_cast<const uint4*>(x + i);
+        uint32_t w[4] = {raw.x, raw.y, raw.z, raw.w};
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            if constexpr (sizeof(T) == 2) {
+                const float lo = fmaxf(__uint_as_float(w[j] << 16), 0.f), hi = fmaxf(__uint_as_float(w[j] & 0xffff0000u), 0.f);
+                w[j] = pack_bf16x2(lo * lo, hi * hi);
+            } else {
+                const float v = fmaxf(__uint_as_float(w[j]), 0.f);
+                w[j] = __float_as_uint(v * v);
+            }
+        }
+        *reinterpret_cast<uint4*>(x + i) = make_uint4(w[0], w[1], w[2], w[3]);
+        return;
+    }
+    for (size_t k = i; k < n; ++k) {
+        const float v = fmaxf(to_f32(x[k]), 0.f);
+        x[k] = from_f32<T>(v * v);
+    }
 }
 
 // ------------------------------------------------------------------ scattered int32 writes
@@ -535,18 +575,36 @@ int llms_scatter_i32(int* dst, const int* index, const int* value, int n, hipStr
     LLMS_LAUNCH_CHECK();
 }
 
-int llms_silu_mul(int dtype, void* out, const void* gate_up, int n_rows, int inter, hipStream_t stream) {
+// clamped: the clamped unit with `limit` instead of SiLU(gate) * up
+int llms_silu_mul(int dtype, void* out, const void* gate_up, int n_rows, int inter, int clamped, float limit,
+                  hipStream_t stream) {
     LLMS_REQUIRE(n_rows > 0 && inter > 0, "silu_mul: sizes must be positive");
     const size_t total = (size_t)n_rows * inter;
     if (dtype == 1 && inter % 8 == 0 && ((uintptr_t)out % 16) == 0 && ((uintptr_t)gate_up % 16) == 0) {
         const size_t chunks = total / 8;
-        silu_mul_bf16_vec_kernel<<<(unsigned)((chunks + 255) / 256), 256, 0, stream>>>((bf16*)out, (const bf16*)gate_up,
-                                                                                         inter, chunks);
+        const unsigned vec_blocks = (unsigned)((chunks + 255) / 256);
+        if (clamped)
+            silu_mul_bf16_vec_kernel<true><<<vec_blocks, 256, 0, stream>>>((bf16*)out, (const bf16*)gate_up, inter, chunks, limit);
+        else
+            silu_mul_bf16_vec_kernel<false><<<vec_blocks, 256, 0, stream>>>((bf16*)out, (const bf16*)gate_up, inter, chunks, limit);
         LLMS_LAUNCH_CHECK();
     }
     const unsigned blocks = (unsigned)((total + 255) / 256);
-    DISPATCH_DTYPE(dtype, silu_mul_kernel<T><<<blocks, 256, 0, stream>>>((T*)out, (const T*)gate_up, inter,
-                                                                          total);)
+    if (clamped) {
+        DISPATCH_DTYPE(dtype, silu_mul_kernel<T, true><<<blocks, 256, 0, stream>>>((T*)out, (const T*)gate_up, inter, total, limit);)
+    } else {
+        DISPATCH_DTYPE(dtype, silu_mul_kernel<T, false><<<blocks, 256, 0, stream>>>((T*)out, (const T*)gate_up, inter, total, limit);)
+    }
+    LLMS_LAUNCH_CHECK();
+}
+
+int llms_squared_relu(int dtype, void* x, size_t n, hipStream_t stream) {
+    LLMS_REQUIRE(n > 0 && ((uintptr_t)x % 16) == 0, "squared_relu: a 16-byte aligned array");
+    DISPATCH_DTYPE(dtype, {
+        const size_t threads = (n + 16 / sizeof(T) - 1) / (16 / sizeof(T));
+        LLMS_REQUIRE((threads + 255) / 256 < (1ull << 31), "squared_relu: too many elements for one launch");
+        squared_relu_kernel<T><<<(unsigned)((threads + 255) / 256), 256, 0, stream>>>((T*)x, n);
+    })
     LLMS_LAUNCH_CHECK();
 }
 

@@ -25,8 +25,9 @@
 // beyond its end, which brings zeros and touches no memory.
 //
 // Epilogues (the waves' partial sums meet in LDS in the order of the waves):
-//   PLAIN     C = sums (+ bias), float32 or bfloat16.
-//   SWIGLU    W = [gate; up]; C[m, f] = bf16(silu(bf16(gate))) * bf16(up)   (src/llmserve/model/llama.py:120).
+//   PLAIN     C = sums (+ bias), float32 or bfloat16; `unit` 2: max(sums, 0)^2.
+//   SWIGLU    W = [gate; up]; C[m, f] = bf16(silu(bf16(gate))) * bf16(up)   (src/llmserve/model/llama.py:120); `unit` 1:
+//             g sigmoid(1.702 g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit), in 32-bit.
 //   ROPE_QKV  W = [q; k; v]; q and k rotated (src/llmserve/model/llama.py:31-54), q written, k and v stored at the
 //             tokens' slots of the paged cache (values transposed inside a page).
 //   RESIDUAL  residual[m, n] = bf16(residual[m, n] + bf16(sums)) in place: the layer's residual sum
@@ -54,6 +55,9 @@ typedef __attribute__((ext_vector_type(4))) unsigned int u32x4;
 #define GD_ROPE_QKV 2
 #define GD_RESIDUAL 3
 
+#define GD_UNIT_CLAMPED 1
+#define GD_UNIT_RELU2 2
+
 struct DecodeGemmArgs {
     const bf16* W;
     const bf16* X;
@@ -69,6 +73,8 @@ struct DecodeGemmArgs {
     int x_rows;     // rows of X kept in LDS: 8 or 16
     int x_pitch;    // bytes from row to row there: all chunks of K and 16 more (rows then start in different banks)
     int inter;  // SWIGLU
+    int unit;   // what is made of the sums: 0 the epilogue's own (SiLU for SWIGLU), 1 the clamped unit, 2 the squared relu
+    float limit;  // of the clamped unit
     int n_heads, n_kv_heads, head_dim, block_size;  // ROPE_QKV
     // ceil(2^32 / (head_dim / 2)): a unit's head by one multiply (exact while unit * head_dim < 2^32, which the
     // entry point checks); log2 of the page size, or -1 if it is no power of 2
@@ -186,6 +192,10 @@ template <typename TOut, int EPI>
 __device__ __forceinline__ void gd_finish_row(const DecodeGemmArgs& a, int m, int n, float s, const GdFinish& f,
                                               size_t part_offset = 0) {
     if (a.bias) s += bf16_bits_to_f32(a.bias[n].bits);
+    if (EPI == GD_PLAIN && a.unit == GD_UNIT_RELU2) {
+        const float r = fmaxf(s, 0.f);
+        s = r * r;
+    }
     if (EPI == GD_PLAIN)
         gd_store<TOut>(reinterpret_cast<TOut*>(a.C) + part_offset + (size_t)m * a.ldc + n, s);
     else
@@ -196,6 +206,11 @@ __device__ __forceinline__ void gd_finish_row(const DecodeGemmArgs& a, int m, in
 template <typename TOut, int EPI>
 __device__ __forceinline__ void gd_finish_pair(const DecodeGemmArgs& a, int m, int u, float lo, float hi, const GdFinish& f) {
     if (EPI == GD_SWIGLU) {
+        if (a.unit == GD_UNIT_CLAMPED) {
+            const float g = fminf(lo, a.limit), v = fminf(fmaxf(hi, -a.limit), a.limit);
+            gd_store<TOut>(reinterpret_cast<TOut*>(a.C) + (size_t)m * a.ldc + u, g / (1.f + expf(-1.702f * g)) * (v + 1.f));
+            return;
+        }
         const float gate = gd_bfr(lo), up = gd_bfr(hi);
         gd_store<TOut>(reinterpret_cast<TOut*>(a.C) + (size_t)m * a.ldc + u, gd_bfr(gate / (1.f + expf(-gate))) * up);
         return;
@@ -822,6 +837,7 @@ int llms_gemm_decode_fits(int M, int K) {
 // `slots` when given; the angles as position times inv_freq, or their sines and cosines as `angles` [M][head_dim / 2][2],
 // or neither: no rotation), 3 residual (residual[M, N] += X W^T in place, bfloat16; C unused).
 // norm_weight (bfloat16 [K]) given: the rows of X are replaced by RMSNorm(X) * norm_weight with `eps` on the way in.
+// unit: 0, or what is made of the sums instead: 1 (gated epilogue) the clamped unit with `limit`, 2 (plain) max(sum, 0)^2.
 // workgroups: how many share the work out (the caller passes the number of compute units).
 // k_parts > 1 (17 to 64 rows, plain 32-bit sums): K is shared out as well, to k_parts sets of workgroups, and C is
 // [k_parts][M][ldc]: partial sums for a norm to add up.
@@ -829,7 +845,7 @@ int llms_gemm_decode(int out_dtype, int epilogue, void* C, int ldc, const void* 
                      const void* bias, const void* norm_weight, float eps, int M, int N, int K, int inter,
                      int n_heads, int n_kv_heads, int head_dim, int block_size, const float* inv_freq,
                      const float* angles, const int* positions, const int* slots, void* k_pool, void* v_pool,
-                     void* residual, int ldr, int workgroups, int k_parts, hipStream_t stream) {
+                     void* residual, int ldr, int workgroups, int k_parts, int unit, float limit, hipStream_t stream) {
     LLMS_REQUIRE(M > 0 && M <= 64 && N > 0 && K > 0, "gemm_decode: needs 1 <= M <= 64 and positive sizes");
     LLMS_REQUIRE((long long)N * K < (1ll << 30) && (long long)M * ldx < (1ll << 30), "gemm_decode: operands of 2 GB or more");
     const int x_rows = M <= 8 ? 8 : 16, x_pitch = (K + GD_KC - 1) / GD_KC * (GD_KC * 2) + 16;
@@ -846,8 +862,10 @@ int llms_gemm_decode(int out_dtype, int epilogue, void* C, int ldc, const void* 
     LLMS_REQUIRE(out_dtype == 1 || (out_dtype == 0 && epilogue == GD_PLAIN), "gemm_decode: 32-bit output goes with the plain epilogue");
     LLMS_REQUIRE(workgroups > 0 && workgroups <= 4096, "gemm_decode: bad number of workgroups");
     DecodeGemmArgs a = {(const bf16*)W, (const bf16*)X, (const bf16*)bias, (const bf16*)norm_weight, eps, C, ldc, ldx,
-                        M, N, K, 0, 0, 0, 0, x_rows, x_pitch, inter, n_heads, n_kv_heads, head_dim, block_size, 0u, -1, inv_freq, angles, positions, slots,
+                        M, N, K, 0, 0, 0, 0, x_rows, x_pitch, inter, unit, limit, n_heads, n_kv_heads, head_dim, block_size, 0u, -1, inv_freq, angles, positions, slots,
                         (bf16*)k_pool, (bf16*)v_pool, (bf16*)residual, ldr, K, 1, K, 0, 0};
+    LLMS_REQUIRE(unit == 0 || (unit == GD_UNIT_CLAMPED && epilogue == GD_SWIGLU) || (unit == GD_UNIT_RELU2 && epilogue == GD_PLAIN && k_parts == 1),
+                 "gemm_decode: the clamped unit goes with the gated epilogue, the squared relu with the plain one");
     if (epilogue == GD_PLAIN) {
         LLMS_REQUIRE(C != nullptr && ldc >= N, "gemm_decode: bad output");
         a.units = N;

@@ -59,8 +59,10 @@ struct StreamArgs {
     int M, N, K;
     int num_tiles;  // tiles of 16 weight rows (8 features for the gated and rotary epilogues)
     int k_splits;   // workgroups that share a tile's K (blockIdx.y); each stores its partial sums, 32-bit, in C[split]
-    // SWIGLU
+    // SWIGLU; unit 1: g sigmoid(1.702 g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit), in 32-bit
     int inter;
+    int unit;
+    float limit;
     // ROPE_QKV
     int n_heads, n_kv_heads, head_dim, block_size;
     const float* inv_freq;
@@ -215,7 +217,13 @@ __global__ __launch_bounds__(NW* LLMS_WAVE) void gemm_stream_kernel(const Stream
     } else if (EPI == EPI_SWIGLU) {
         const int j = idx % 8, ml = idx / 8, m = m0 + ml, f = tile_id * 8 + j;
         if (idx < 128 && m < M && f < a.inter) {
-            const float gate = bfr(total_of(j, ml)), up = bfr(total_of(j + 8, ml));
+            const float lo = total_of(j, ml), hi = total_of(j + 8, ml);
+            if (a.unit == 1) {
+                const float gc = fminf(lo, a.limit), uc = fminf(fmaxf(hi, -a.limit), a.limit);
+                store_out<TOut>(C + (size_t)m * a.ldc + f, gc / (1.f + expf(-1.702f * gc)) * (uc + 1.f));
+                return;
+            }
+            const float gate = bfr(lo), up = bfr(hi);
             store_out<TOut>(C + (size_t)m * a.ldc + f, bfr(gate / (1.f + expf(-gate))) * up);
         }
     } else {
@@ -365,7 +373,7 @@ extern "C" {
 int llms_gemm_stream(int out_dtype, int epilogue, void* C, int ldc, const void* X, int ldx, const void* W,
                      const void* bias, int M, int N, int K, int inter, int n_heads, int n_kv_heads, int head_dim,
                      int block_size, const float* inv_freq, const int* positions, const int* slots, void* k_pool,
-                     void* v_pool, int k_splits, hipStream_t stream) {
+                     void* v_pool, int k_splits, int unit, float limit, hipStream_t stream) {
     LLMS_REQUIRE(M > 0 && M <= 64 && N > 0 && K > 0, "gemm_stream: needs 1 <= M <= 64 and positive sizes");
     LLMS_REQUIRE(K % 8 == 0 && ldx % 8 == 0 && ldx >= K, "gemm_stream: K and the row stride of X must be multiples of 8");
     LLMS_REQUIRE(((uintptr_t)X % 16) == 0 && ((uintptr_t)W % 16) == 0, "gemm_stream: X and W must be 16-byte aligned");
@@ -374,8 +382,9 @@ int llms_gemm_stream(int out_dtype, int epilogue, void* C, int ldc, const void* 
     LLMS_REQUIRE(k_splits >= 1 && k_splits <= 16, "gemm_stream: k_splits must be in 1..16");
     LLMS_REQUIRE(k_splits == 1 || (epilogue == EPI_PLAIN && out_dtype == 0),
                  "gemm_stream: K is split for plain 32-bit partial sums only");
-    StreamArgs a = {C, ldc, (const bf16*)X, ldx, (const bf16*)W, (const bf16*)bias, M, N, K, 0, k_splits, inter, n_heads,
+    StreamArgs a = {C, ldc, (const bf16*)X, ldx, (const bf16*)W, (const bf16*)bias, M, N, K, 0, k_splits, inter, unit, limit, n_heads,
                     n_kv_heads, head_dim, block_size, inv_freq, positions, slots, (bf16*)k_pool, (bf16*)v_pool};
+    LLMS_REQUIRE(unit == 0 || (unit == 1 && epilogue == EPI_SWIGLU), "gemm_stream: the clamped unit goes with the gated epilogue");
     unsigned grid;
     if (epilogue == EPI_PLAIN) {
         LLMS_REQUIRE(ldc >= N, "gemm_stream: ldc too small");

@@ -7,7 +7,8 @@
 // rows of a, then the 32 rows of b of the same units, so that a thread or lane holds both of a unit):
 // out[m, u] = min(a, limit) * sigmoid(1.702 min(a, limit)) * (clamp(b, -limit, limit) + 1) for the `units` units
 // (unit 0), or a * sigmoid(a) * b (unit 1);
-// "gated": the result times sigmoid(z[m, g * z_gs + n]) with z in 32-bit.
+// "gated": the result times sigmoid(z[m, g * z_gs + n * z_ns]) with z in 32-bit (z_ns 1: a gate per element; 0: one number
+// for a row of a group).
 // Two kernels: 32-bit multiply-add (any sizes, float or bfloat16 operands, 32-bit products and sums) and bfloat16 on
 // the matrix cores (K and the strides of x in multiples of 8, 16-byte aligned operands).
 #include "common.h"
@@ -40,7 +41,7 @@ template <typename TIn, typename TOut, int EPI>
 __global__ __launch_bounds__(256) void grouped_fma_kernel(
     TOut* __restrict__ out, long out_ld, long out_gs, const TIn* __restrict__ x, long x_ld, long x_gs,
     const TIn* __restrict__ w, int M, int N, int K, int G, const int* __restrict__ seg, const int* __restrict__ tile_start,
-    const float* __restrict__ z, long z_ld, long z_gs, float limit, int unit, int units) {
+    const float* __restrict__ z, long z_ld, long z_gs, int z_ns, float limit, int unit, int units) {
     __shared__ float As[GG_TK][GG_TM + 4];
     __shared__ float Ws[GG_TK][GG_TN + 4];
     const int tid = threadIdx.x;
@@ -106,7 +107,7 @@ __global__ __launch_bounds__(256) void grouped_fma_kernel(
                 const int n = n0 + column(j);
                 if (n >= N) continue;
                 float v = acc[i][j];
-                if (EPI == GG_GATED) v = v / (1.f + expf(-z[(size_t)m * z_ld + (size_t)g * z_gs + n]));
+                if (EPI == GG_GATED) v = v / (1.f + expf(-z[(size_t)m * z_ld + (size_t)g * z_gs + (size_t)n * z_ns]));
                 og[(size_t)m * out_ld + n] = from_f32<TOut>(v);
             }
         }
@@ -116,10 +117,10 @@ __global__ __launch_bounds__(256) void grouped_fma_kernel(
 template <typename TIn, typename TOut>
 static int launch_fma(int epilogue, dim3 grid, hipStream_t stream, void* out, long out_ld, long out_gs, const void* x, long x_ld,
                       long x_gs, const void* w, int M, int N, int K, int G, const int* seg, const int* tile_start, const float* z,
-                      long z_ld, long z_gs, float limit, int unit, int units) {
+                      long z_ld, long z_gs, int z_ns, float limit, int unit, int units) {
 #define GG_GO(EPI)                                                                                                          \
     grouped_fma_kernel<TIn, TOut, EPI><<<grid, 256, 0, stream>>>((TOut*)out, out_ld, out_gs, (const TIn*)x, x_ld, x_gs,      \
-                                                                 (const TIn*)w, M, N, K, G, seg, tile_start, z, z_ld, z_gs, limit, unit, units)
+                                                                 (const TIn*)w, M, N, K, G, seg, tile_start, z, z_ld, z_gs, z_ns, limit, unit, units)
     if (epilogue == GG_PLAIN) GG_GO(GG_PLAIN);
     else if (epilogue == GG_PAIRED) GG_GO(GG_PAIRED);
     else GG_GO(GG_GATED);
@@ -148,7 +149,7 @@ template <typename TOut, int EPI>
 __global__ __launch_bounds__(256) void grouped_mfma_kernel(
     TOut* __restrict__ out, long out_ld, long out_gs, const bf16* __restrict__ x, long x_ld, long x_gs,
     const bf16* __restrict__ w, int M, int N, int K, int G, const int* __restrict__ seg, const int* __restrict__ tile_start,
-    const float* __restrict__ z, long z_ld, long z_gs, float limit, int unit, int units, int k_part, long part_stride) {
+    const float* __restrict__ z, long z_ld, long z_gs, int z_ns, float limit, int unit, int units, int k_part, long part_stride) {
     extern __shared__ __attribute__((aligned(16))) uint16_t gm_lds[];
     uint16_t(*As)[GM_BM * GM_LD] = reinterpret_cast<uint16_t(*)[GM_BM * GM_LD]>(gm_lds);
     uint16_t(*Bs)[GM_BN * GM_LD] = reinterpret_cast<uint16_t(*)[GM_BN * GM_LD]>(gm_lds + 2 * GM_BM * GM_LD);
@@ -251,7 +252,7 @@ __global__ __launch_bounds__(256) void grouped_mfma_kernel(
                     const int n = n0 + wn + j * 32 + l32;
                     if (n >= N) continue;
                     float v = acc[i][j][r];
-                    if (EPI == GG_GATED) v = v / (1.f + expf(-z[(size_t)m * z_ld + (size_t)g * z_gs + n]));
+                    if (EPI == GG_GATED) v = v / (1.f + expf(-z[(size_t)m * z_ld + (size_t)g * z_gs + (size_t)n * z_ns]));
                     og[(size_t)m * out_ld + n] = from_f32<TOut>(v);
                 }
             }
@@ -262,12 +263,12 @@ __global__ __launch_bounds__(256) void grouped_mfma_kernel(
 template <typename TOut>
 static int launch_mfma(int epilogue, dim3 grid, hipStream_t stream, void* out, long out_ld, long out_gs, const void* x, long x_ld,
                        long x_gs, const void* w, int M, int N, int K, int G, const int* seg, const int* tile_start, const float* z,
-                       long z_ld, long z_gs, float limit, int unit, int units, int k_part, long part_stride) {
+                       long z_ld, long z_gs, int z_ns, float limit, int unit, int units, int k_part, long part_stride) {
 #define GM_GO(EPI)                                                                                                          \
     LLMS_HIP_CHECK(hipFuncSetAttribute((const void*)grouped_mfma_kernel<TOut, EPI>,                                         \
                                        hipFuncAttributeMaxDynamicSharedMemorySize, GM_LDS_BYTES));                          \
     grouped_mfma_kernel<TOut, EPI><<<grid, 256, GM_LDS_BYTES, stream>>>((TOut*)out, out_ld, out_gs, (const bf16*)x, x_ld, x_gs, \
-                                                             (const bf16*)w, M, N, K, G, seg, tile_start, z, z_ld, z_gs, limit, unit, units, \
+                                                             (const bf16*)w, M, N, K, G, seg, tile_start, z, z_ld, z_gs, z_ns, limit, unit, units, \
                                                              k_part, part_stride)
     if (epilogue == GG_PLAIN) {
         GM_GO(GG_PLAIN);
@@ -287,7 +288,7 @@ extern "C" {
 // tile_start[G], which the host bounds by ceil(M / 64) + G).
 int llms_grouped_fma(int in_dtype, int out_dtype, int epilogue, void* out, long out_ld, long out_gs, const void* x, long x_ld,
                      long x_gs, const void* w, int M, int N, int K, int G, const int* seg, const int* tile_start,
-                     int max_tiles, const float* z, long z_ld, long z_gs, float limit, int unit, int units, hipStream_t stream) {
+                     int max_tiles, const float* z, long z_ld, long z_gs, int z_ns, float limit, int unit, int units, hipStream_t stream) {
     LLMS_REQUIRE(M > 0 && N > 0 && K > 0 && G > 0, "grouped_fma: sizes must be positive");
     LLMS_REQUIRE(epilogue >= 0 && epilogue <= 2, "grouped_fma: epilogue 0 (plain), 1 (paired) or 2 (gated)");
     LLMS_REQUIRE(epilogue != GG_PAIRED || (N % 64 == 0 && units > 0 && units <= N / 2),
@@ -298,13 +299,13 @@ int llms_grouped_fma(int in_dtype, int out_dtype, int epilogue, void* out, long 
     LLMS_REQUIRE(grid.y > 0 && grid.y <= 65535 && grid.z <= 65535, "grouped_fma: too many rows or groups for one launch");
     if (in_dtype == 0 && out_dtype == 0)
         return launch_fma<float, float>(epilogue, grid, stream, out, out_ld, out_gs, x, x_ld, x_gs, w, M, N, K, G, seg, tile_start,
-                                        z, z_ld, z_gs, limit, unit, units);
+                                        z, z_ld, z_gs, z_ns, limit, unit, units);
     if (in_dtype == 1 && out_dtype == 1)
         return launch_fma<bf16, bf16>(epilogue, grid, stream, out, out_ld, out_gs, x, x_ld, x_gs, w, M, N, K, G, seg, tile_start, z,
-                                      z_ld, z_gs, limit, unit, units);
+                                      z_ld, z_gs, z_ns, limit, unit, units);
     if (in_dtype == 1 && out_dtype == 0)
         return launch_fma<bf16, float>(epilogue, grid, stream, out, out_ld, out_gs, x, x_ld, x_gs, w, M, N, K, G, seg, tile_start, z,
-                                       z_ld, z_gs, limit, unit, units);
+                                       z_ld, z_gs, z_ns, limit, unit, units);
     LLMS_REQUIRE(false, "grouped_fma: unsupported dtype pair");
 }
 
@@ -313,7 +314,7 @@ int llms_grouped_fma(int in_dtype, int out_dtype, int epilogue, void* out, long 
 // leaving its sums at out + p * part_stride.
 int llms_grouped_mfma(int out_dtype, int epilogue, void* out, long out_ld, long out_gs, const void* x, long x_ld, long x_gs,
                       const void* w, int M, int N, int K, int G, const int* seg, const int* tile_start, int max_tiles,
-                      const float* z, long z_ld, long z_gs, float limit, int unit, int units, int k_parts, long part_stride,
+                      const float* z, long z_ld, long z_gs, int z_ns, float limit, int unit, int units, int k_parts, long part_stride,
                       hipStream_t stream) {
     LLMS_REQUIRE(M > 0 && N > 0 && K > 0 && G > 0, "grouped_mfma: sizes must be positive");
     LLMS_REQUIRE(epilogue >= 0 && epilogue <= 2, "grouped_mfma: epilogue 0 (plain), 1 (paired) or 2 (gated)");
@@ -331,10 +332,10 @@ int llms_grouped_mfma(int out_dtype, int epilogue, void* out, long out_ld, long 
     LLMS_REQUIRE(grid.y > 0 && grid.y <= 65535 && grid.z <= 65535, "grouped_mfma: too many rows or groups for one launch");
     if (out_dtype == 0)
         return launch_mfma<float>(epilogue, grid, stream, out, out_ld, out_gs, x, x_ld, x_gs, w, M, N, K, G, seg, tile_start, z, z_ld,
-                                  z_gs, limit, unit, units, k_part, part_stride);
+                                  z_gs, z_ns, limit, unit, units, k_part, part_stride);
     if (out_dtype == 1)
         return launch_mfma<bf16>(epilogue, grid, stream, out, out_ld, out_gs, x, x_ld, x_gs, w, M, N, K, G, seg, tile_start, z, z_ld,
-                                 z_gs, limit, unit, units, k_part, part_stride);
+                                 z_gs, z_ns, limit, unit, units, k_part, part_stride);
     LLMS_REQUIRE(false, "grouped_mfma: out_dtype must be 0 or 1");
 }
 

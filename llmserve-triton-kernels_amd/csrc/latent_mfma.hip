@@ -42,6 +42,7 @@ struct LatentArgs {
     int table_width, heads, r, dk, dkp, block_size, window, splits;
     uint32_t page_magic;  // ceil(2^32 / block_size): key / block_size is the high word of key * page_magic (0: block_size is 1)
     float scale_log2;
+    const float* sink;  // [H]: head h's denominator holds one more term, exp(sink[h]), that has no value (null: none)
 };
 
 template <int RT>
@@ -261,6 +262,7 @@ __global__ __launch_bounds__(LM_THREADS) void attend_latent_mfma_kernel(LatentAr
         }
         return;
     }
+    if (a.sink) l += __builtin_amdgcn_exp2f(a.sink[head] * 1.4426950408889634f - m);
     const float inv = l > 0.f ? 1.f / l : 0.f;
     bf16* orow = a.out + row * a.r;
 #pragma unroll
@@ -273,8 +275,10 @@ __global__ __launch_bounds__(LM_THREADS) void attend_latent_mfma_kernel(LatentAr
 // grid: (token, head) pairs; adds the shares up in their order.  Every thread reads the shares' maxima and sums at
 // once (all loads asked for before the first is used), then its numbers of every share.
 #define LM_MAX_SPLITS 16
-__global__ __launch_bounds__(256) void latent_merge_kernel(bf16* __restrict__ out, const float* __restrict__ ws, int r, int splits) {
+__global__ __launch_bounds__(256) void latent_merge_kernel(bf16* __restrict__ out, const float* __restrict__ ws, int r, int splits,
+                                                           const float* __restrict__ sink, int heads) {
     const size_t row = blockIdx.x;
+    const float sink_log2 = sink ? sink[blockIdx.x % heads] * 1.4426950408889634f : -INFINITY;
     const float* shares = ws + row * splits * (r + 2);
     float mz[LM_MAX_SPLITS], lz[LM_MAX_SPLITS];
 #pragma unroll
@@ -291,6 +295,7 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(bf16* __restrict__ ou
         mz[z] = mz[z] > -INFINITY ? __builtin_amdgcn_exp2f(mz[z] - top) : 0.f;  // (from here on: the share's factor)
         total += lz[z] * mz[z];
     }
+    if (sink) total += __builtin_amdgcn_exp2f(sink_log2 - top);
     const float inv = total > 0.f ? 1.f / total : 0.f;
     for (int c = threadIdx.x; c < r; c += 256) {
         float part[LM_MAX_SPLITS];
@@ -327,7 +332,7 @@ int llms_attend_latent_mfma_class(int r, int dk) {
 int llms_attend_latent_mfma(void* out, const void* q, const void* pool, const int* tables, int table_width,
                             const int* table_rows, const int* cu_seqlens, const int* context_lens, float* ws, int n_seqs,
                             int n_rows, int max_count, int heads, int r, int dr, int block_size, int window, float scale,
-                            int splits, hipStream_t stream) {
+                            int splits, const float* sink, hipStream_t stream) {
     LLMS_REQUIRE(n_seqs > 0 && n_rows > 0 && max_count > 0 && heads > 0 && block_size > 0 && table_width > 0,
                  "attend_latent_mfma: sizes must be positive");
     const int dk = r + dr, rt = llms_attend_latent_mfma_class(r, dk);
@@ -341,6 +346,7 @@ int llms_attend_latent_mfma(void* out, const void* q, const void* pool, const in
     a.table_width = table_width, a.heads = heads, a.r = r, a.dk = dk, a.dkp = (dk + 31) / 32 * 32;
     a.block_size = block_size, a.window = window, a.splits = splits;
     a.scale_log2 = scale * 1.4426950408889634f;
+    a.sink = sink;
     a.page_magic = block_size == 1 ? 0u : (uint32_t)(((1ull << 32) + block_size - 1) / block_size);
     const long long blocks = ((long long)max_count * heads + LM_PAIRS - 1) / LM_PAIRS;
     LLMS_REQUIRE(blocks < (1ll << 31) && n_seqs <= 65535, "attend_latent_mfma: too many workgroups for one launch");
@@ -350,7 +356,7 @@ int llms_attend_latent_mfma(void* out, const void* q, const void* pool, const in
                  : rt == 16 ? launch_latent<16>(a, grid, lds, stream)
                             : launch_latent<32>(a, grid, lds, stream);
     if (status != LLMS_OK) return status;
-    if (splits > 1) latent_merge_kernel<<<(unsigned)((size_t)n_rows * heads), 256, 0, stream>>>((bf16*)out, ws, r, splits);
+    if (splits > 1) latent_merge_kernel<<<(unsigned)((size_t)n_rows * heads), 256, 0, stream>>>((bf16*)out, ws, r, splits, sink, heads);
     LLMS_LAUNCH_CHECK();
 }
 

@@ -3,6 +3,8 @@
 //                 wins a tie), in descending order; weight = score or score / (sum of the chosen scores + renorm_eps).
 //                 With `groups` > 1 the experts form that many equal groups of neighbours, a group's score is its largest
 //                 score, and only experts of the `keep` best groups (the lower group wins a tie) can be chosen.
+//                 With a `correction` per expert the choice (groups included) is made on score + correction, the weights
+//                 stay the scores; every weight is multiplied by `weight_scale`.
 //                 `bias` is added to z; `extra` rows of W_router behind the experts' give extra_out = their products
 //   moe_rank      for expert e: how many (token, choice) pairs chose it, and each such pair's rank among them in the
 //                 order of the pairs (so the sorted order is stable and the same whatever runs beside it)
@@ -22,8 +24,10 @@ template <typename T>
 __global__ __launch_bounds__(MOE_THREADS) void moe_router_kernel(
     int* __restrict__ chosen, float* __restrict__ weight, const T* __restrict__ h, const T* __restrict__ w_router,
     int hidden, int experts, int top, int renormalize, int softmax, int groups, int keep, float renorm_eps,
-    const float* __restrict__ bias, int extra, float* __restrict__ extra_out) {
-    extern __shared__ float score[];  // experts, then groups
+    const float* __restrict__ bias, int extra, float* __restrict__ extra_out, const float* __restrict__ correction,
+    float weight_scale) {
+    extern __shared__ float score[];  // experts, then groups, then with a correction what the choice is made on
+    float* choice = correction ? score + experts + groups : score;
     const int n = blockIdx.x, lane = threadIdx.x % LLMS_WAVE, wave = threadIdx.x / LLMS_WAVE;
     const T* row = h + (size_t)n * hidden;
     const bool vec = hidden % (16 / sizeof(T)) == 0 && ((uintptr_t)h % 16) == 0 && ((uintptr_t)w_router % 16) == 0;
@@ -61,7 +65,11 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_router_kernel(
         if (bias) dot += bias[e];
         // (a row that is not a number, as a padding row may be, gets a score like any other: every choice below must
         // name an expert that exists)
-        if (lane == 0) score[e] = dot == dot ? (softmax ? dot : 1.f / (1.f + expf(-dot))) : 0.f;
+        if (lane == 0) {
+            const float s = dot == dot ? (softmax ? dot : 1.f / (1.f + expf(-dot))) : 0.f;
+            score[e] = s;
+            if (correction && !softmax) choice[e] = s + correction[e];
+        }
     }
     __syncthreads();
     if (wave != 0) return;
@@ -76,7 +84,11 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_router_kernel(
             total += w;
         }
         total = wave_sum(total);
-        for (int e = lane; e < experts; e += LLMS_WAVE) score[e] = score[e] / total;
+        for (int e = lane; e < experts; e += LLMS_WAVE) {
+            const float s = score[e] / total;
+            score[e] = s;
+            if (correction) choice[e] = s + correction[e];
+        }
         __builtin_amdgcn_s_waitcnt(0);
         __builtin_amdgcn_wave_barrier();
     }
@@ -84,14 +96,14 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_router_kernel(
         float* best_of = score + experts;
         const int per = experts / groups;
         for (int g = lane; g < groups; g += LLMS_WAVE) {
-            float b = -1.f;
-            for (int e = g * per; e < (g + 1) * per; ++e) b = fmaxf(b, score[e]);
+            float b = -INFINITY;
+            for (int e = g * per; e < (g + 1) * per; ++e) b = fmaxf(b, choice[e]);
             best_of[g] = b;
         }
         __builtin_amdgcn_s_waitcnt(0);
         __builtin_amdgcn_wave_barrier();
         for (int k = 0; k < keep; ++k) {
-            float best = -1.f;
+            float best = -INFINITY;
             int at = 0x7fffffff;
             for (int g = lane; g < groups; g += LLMS_WAVE) {
                 const float b = best_of[g];
@@ -110,12 +122,12 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_router_kernel(
                 }
             }
             at = min(at, groups - 1);
-            if (lane == 0) best_of[at] = -3.f;  // kept
+            if (lane == 0) best_of[at] = -INFINITY;  // kept (no group's best is that low)
             __builtin_amdgcn_s_waitcnt(0);
             __builtin_amdgcn_wave_barrier();
         }
         for (int e = lane; e < experts; e += LLMS_WAVE)
-            if (best_of[e / per] != -3.f) score[e] = -2.f;
+            if (best_of[e / per] != -INFINITY) choice[e] = -INFINITY;
         __builtin_amdgcn_s_waitcnt(0);
         __builtin_amdgcn_wave_barrier();
     }
@@ -123,10 +135,10 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_router_kernel(
     int which[MOE_MAX_TOP];
     float sum = 0.f;
     for (int k = 0; k < top; ++k) {
-        float best = -1.f;  // (scores are in (0, 1); a taken expert is marked -2)
+        float best = -INFINITY;  // (what a taken expert is marked with)
         int at = 0x7fffffff;
         for (int e = lane; e < experts; e += LLMS_WAVE) {
-            const float s = score[e];
+            const float s = choice[e];
             if (s > best) {
                 best = s;
                 at = e;
@@ -142,17 +154,18 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_router_kernel(
             }
         }
         at = min(at, experts - 1);
+        if (correction) best = score[at];
         picked[k] = best;
         which[k] = at;
         sum += best;
-        if (lane == 0) score[at] = -2.f;
+        if (lane == 0) choice[at] = -INFINITY;
         __builtin_amdgcn_s_waitcnt(0);
         __builtin_amdgcn_wave_barrier();
     }
     if (lane == 0)
         for (int k = 0; k < top; ++k) {
             chosen[(size_t)n * top + k] = which[k];
-            weight[(size_t)n * top + k] = renormalize ? picked[k] / (sum + renorm_eps) : picked[k];
+            weight[(size_t)n * top + k] = weight_scale * (renormalize ? picked[k] / (sum + renorm_eps) : picked[k]);
         }
 }
 
@@ -329,7 +342,7 @@ extern "C" {
 
 int llms_moe_router(int dtype, int* chosen, float* weight, const void* h, const void* w_router, int n, int hidden, int experts,
                     int top, int renormalize, int softmax, int groups, int keep, float renorm_eps, const float* bias, int extra,
-                    float* extra_out, hipStream_t stream) {
+                    float* extra_out, const float* correction, float weight_scale, hipStream_t stream) {
     LLMS_REQUIRE(n > 0 && hidden > 0 && experts > 0, "moe_router: sizes must be positive");
     LLMS_REQUIRE(extra >= 0 && (extra == 0 || extra_out), "moe_router: extra rows need a place for their products");
     LLMS_REQUIRE(top >= 1 && top <= MOE_MAX_TOP && top <= experts, "moe_router: 1 to 16 choices, no more than there are experts");
@@ -338,13 +351,15 @@ int llms_moe_router(int dtype, int* chosen, float* weight, const void* h, const 
     LLMS_REQUIRE(groups >= 1 && experts % groups == 0 && keep >= 1 && keep <= groups,
                  "moe_router: the groups must share the experts out equally, and 1 to all of them are kept");
     LLMS_REQUIRE(groups == 1 || top <= keep * (experts / groups), "moe_router: the kept groups hold fewer experts than are chosen");
-    const size_t lds = (size_t)(experts + groups) * sizeof(float);
+    const size_t lds = (size_t)(experts + groups + (correction ? experts : 0)) * sizeof(float);
     if (dtype == 0)
         moe_router_kernel<float><<<n, MOE_THREADS, lds, stream>>>(chosen, weight, (const float*)h, (const float*)w_router, hidden,
-                                                                  experts, top, renormalize, softmax, groups, keep, renorm_eps, bias, extra, extra_out);
+                                                                  experts, top, renormalize, softmax, groups, keep, renorm_eps, bias, extra, extra_out,
+                                                                  correction, weight_scale);
     else
         moe_router_kernel<bf16><<<n, MOE_THREADS, lds, stream>>>(chosen, weight, (const bf16*)h, (const bf16*)w_router, hidden,
-                                                                 experts, top, renormalize, softmax, groups, keep, renorm_eps, bias, extra, extra_out);
+                                                                 experts, top, renormalize, softmax, groups, keep, renorm_eps, bias, extra, extra_out,
+                                                                  correction, weight_scale);
     LLMS_LAUNCH_CHECK();
 }
 

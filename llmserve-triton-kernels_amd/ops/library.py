@@ -242,8 +242,9 @@ def scatter_i32(dst: torch.Tensor, index: torch.Tensor, value: torch.Tensor) -> 
                                                 _stream(dev)), "scatter_i32")
 
 
-def silu_mul(out: torch.Tensor, gate_up: torch.Tensor) -> torch.Tensor:
-    """out = silu(gate_up[:, :I]) * gate_up[:, I:]."""
+def silu_mul(out: torch.Tensor, gate_up: torch.Tensor, limit: float | None = None) -> torch.Tensor:
+    """out = silu(gate_up[:, :I]) * gate_up[:, I:]; with `limit` g sigmoid(1.702 g) (u + 1), g = min(gate, limit),
+    u = clamp(up, -limit, limit)."""
     dev = _dev(out, gate_up)
     _rows(out, "out")
     _rows(gate_up, "gate_up", 2 * out.shape[1])
@@ -252,9 +253,20 @@ def silu_mul(out: torch.Tensor, gate_up: torch.Tensor) -> torch.Tensor:
     if out.shape[0] == 0:
         return out
     _check(load("elementwise").llms_silu_mul(
-        c_int(_code(out)), _ptr(out), _ptr(gate_up), c_int(out.shape[0]), c_int(out.shape[1]), _stream(dev)),
-        "silu_mul")
+        c_int(_code(out)), _ptr(out), _ptr(gate_up), c_int(out.shape[0]), c_int(out.shape[1]), c_int(limit is not None),
+        c_float(limit or 0.0), _stream(dev)), "silu_mul")
     return out
+
+
+def squared_relu(x: torch.Tensor) -> torch.Tensor:
+    """x <- max(x, 0)^2 in place; x contiguous, 16-byte aligned."""
+    dev = _dev(x)
+    if not x.is_contiguous() or x.data_ptr() % 16:
+        raise ValueError("x must be contiguous and 16-byte aligned")
+    if x.numel():
+        _check(load("elementwise").llms_squared_relu(c_int(_code(x)), _ptr(x), ctypes.c_size_t(x.numel()), _stream(dev)),
+               "squared_relu")
+    return x
 
 
 # ------------------------------------------------------------------------------ matrix products
@@ -326,11 +338,11 @@ def gemm_bf16(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor, bias: torch.T
 
 
 def gemm_stream(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None, *,
-                swiglu: bool = False, rope: dict | None = None, k_splits: int = 1) -> torch.Tensor:
+                swiglu: bool = False, rope: dict | None = None, k_splits: int = 1, limit: float | None = None) -> torch.Tensor:
     """The product for up to 64 bfloat16 rows (built for up to 16), with what surrounds it fused in.
 
     plain:   out[M, N] = x w^T (+ bias).
-    swiglu:  w = [gate; up] ([2I, K]); out[M, I] = silu(gate) * up.
+    swiglu:  w = [gate; up] ([2I, K]); out[M, I] = silu(gate) * up, or with `limit` the clamped unit of `silu_mul`.
     rope = dict(n_heads, n_kv_heads, head_dim, inv_freq | None, positions, slots | None, k_pool, v_pool,
              block_size): w = [q; k; v]; out[M, n_heads * head_dim] = rotated q; rotated k and v are stored at
              the tokens' cache slots.
@@ -357,8 +369,8 @@ def gemm_stream(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor, bias: torch
                          "and 16-byte aligned operands")
     if bias is not None and (bias.dtype != torch.bfloat16 or bias.numel() != n or not bias.is_contiguous()):
         raise ValueError("bias must be a contiguous bfloat16 vector of N elements")
-    if swiglu and rope is not None:
-        raise ValueError("one epilogue at a time")
+    if (swiglu and rope is not None) or (limit is not None and not swiglu):
+        raise ValueError("one epilogue at a time; a limit goes with the gated one")
     epilogue, inter, cols = 0, 0, n
     r = dict(n_heads=0, n_kv_heads=0, head_dim=0, block_size=0, inv_freq=None, positions=None, slots=None,
              k_pool=None, v_pool=None, angles=None)
@@ -391,7 +403,7 @@ def gemm_stream(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor, bias: torch
         c_int(_code(out)), c_int(epilogue), _ptr(out), c_int(out.stride(0)), _ptr(x), c_int(x.stride(0)), _ptr(w),
         _ptr(bias), c_int(m), c_int(n), c_int(k), c_int(inter), c_int(r["n_heads"]), c_int(r["n_kv_heads"]), c_int(r["head_dim"]), c_int(r["block_size"]),
         _ptr(r["inv_freq"]), _ptr(r["positions"]), _ptr(r["slots"]), _ptr(r["k_pool"]), _ptr(r["v_pool"]),
-        c_int(k_splits), _stream(dev)), "gemm_stream")
+        c_int(k_splits), c_int(limit is not None), c_float(limit or 0.0), _stream(dev)), "gemm_stream")
     return parts if k_splits != 1 else out
 
 
@@ -447,12 +459,14 @@ def gemm_decode_supported(x: torch.Tensor, w: torch.Tensor) -> bool:
 
 def gemm_decode(out: torch.Tensor | None, x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None, *,
                 norm: tuple[torch.Tensor, float] | None = None, swiglu: bool = False, rope: dict | None = None,
-                residual: torch.Tensor | None = None, k_parts: int = 1) -> torch.Tensor:
+                residual: torch.Tensor | None = None, k_parts: int = 1, limit: float | None = None,
+                squared_relu: bool = False) -> torch.Tensor:
     """The product for up to 64 bfloat16 rows with one workgroup per compute unit, and what surrounds it fused in.
 
     norm = (weight [K], eps): the rows of x are replaced by RMSNorm(x) * weight on the way in (up to 16 rows).
-    plain:     out[M, N] = x w^T (+ bias), bfloat16 or float32.
-    swiglu:    w = [gate; up] ([2I, K]); out[M, I] = silu(gate) * up.
+    plain:     out[M, N] = x w^T (+ bias), bfloat16 or float32; `squared_relu`: max(x w^T, 0)^2.
+    swiglu:    w = [gate; up] ([2I, K]); out[M, I] = silu(gate) * up, or with `limit` the clamped unit of `silu_mul`
+               (in 32-bit, rounded once).
     rope = dict(n_heads, n_kv_heads, head_dim, inv_freq | None, positions, slots | None, k_pool, v_pool,
                block_size, angles | None): w = [q; k; v]; out[M, n_heads * head_dim] = rotated q; rotated k and v
                are stored at the tokens' cache slots.  `angles` (rotary_angles(positions, inv_freq), float32
@@ -490,6 +504,8 @@ def gemm_decode(out: torch.Tensor | None, x: torch.Tensor, w: torch.Tensor, bias
         raise ValueError("bias must be a contiguous bfloat16 vector of N elements")
     if sum((swiglu, rope is not None, residual is not None)) > 1:
         raise ValueError("one epilogue at a time")
+    if (limit is not None and not swiglu) or (squared_relu and (swiglu or rope is not None or residual is not None or k_parts > 1)):
+        raise ValueError("a limit goes with the gated epilogue, the squared relu with the plain one (K not shared out)")
     norm_weight, eps = None, 0.0
     if norm is not None:
         norm_weight, eps = norm
@@ -541,7 +557,7 @@ def gemm_decode(out: torch.Tensor | None, x: torch.Tensor, w: torch.Tensor, bias
         c_int(r["n_kv_heads"]), c_int(r["head_dim"]), c_int(r["block_size"]), _ptr(r["inv_freq"]), _ptr(r["angles"]), _ptr(r["positions"]),
         _ptr(r["slots"]), _ptr(r["k_pool"]), _ptr(r["v_pool"]), _ptr(residual),
         c_int(residual.stride(0) if residual is not None else 0), c_int(compute_units(dev)), c_int(k_parts),
-        _stream(dev)), "gemm_decode")
+        c_int(1 if limit is not None else 2 if squared_relu else 0), c_float(limit or 0.0), _stream(dev)), "gemm_decode")
     return residual if epilogue == 3 else out
 
 
@@ -677,7 +693,8 @@ def attention_mfma(out: torch.Tensor, q: torch.Tensor, k_pool: torch.Tensor, v_p
                    seq_begin: int, n_seqs: int, max_new: int, token_begin: int, n_tokens: int,
                    n_heads: int, n_kv_heads: int, head_dim: int, block_size: int, window: int = 0,
                    scale: float | None = None, split_waves: bool = False, num_splits: int = 1,
-                   table_rows: torch.Tensor | None = None, waves: int = 4, merge_kernel: bool = False) -> torch.Tensor:
+                   table_rows: torch.Tensor | None = None, waves: int = 4, merge_kernel: bool = False,
+                   head_gate: torch.Tensor | None = None) -> torch.Tensor:
     """bfloat16 causal attention on the matrix cores for requests [seq_begin, seq_begin + n_seqs) of a
     step, whose new tokens are rows [token_begin, token_begin + n_tokens) of q and out and bring at most
     `max_new` tokens each.  `split_waves` (with `waves` = 4 or 8 and `num_splits`) spreads each request's keys
@@ -687,8 +704,10 @@ def attention_mfma(out: torch.Tensor, q: torch.Tensor, k_pool: torch.Tensor, v_p
     shares the keys of such a block of tokens out to several workgroups (short portions, long prefixes).
     The shares of workgroups are added up, in the order of the splits, by a second kernel, or for decoding with up
     to 16 splits by the workgroup of each group that finishes last (`merge_kernel=True` asks for the second kernel
-    there too: the same bits).  (For prompt portions the last workgroup was tried as well: no faster.)"""
-    dev = _dev(out, q, k_pool, v_pool, block_tables, cu_seqlens, context_lens, table_rows)
+    there too: the same bits).  (For prompt portions the last workgroup was tried as well: no faster.)
+    `head_gate` float32 [N, >= n_heads] (unit inner stride): every head's result is multiplied by the sigmoid of the
+    token's number for it."""
+    dev = _dev(out, q, k_pool, v_pool, block_tables, cu_seqlens, context_lens, table_rows, head_gate)
     _check_paged(q, out, k_pool, v_pool, block_tables, n_heads, n_kv_heads, head_dim, block_size)
     if not attention_mfma_supported(q.dtype, head_dim, block_size):
         raise ValueError(f"attention_mfma needs bfloat16, head_dim a multiple of 16 up to 256 and block_size a "
@@ -712,6 +731,9 @@ def attention_mfma(out: torch.Tensor, q: torch.Tensor, k_pool: torch.Tensor, v_p
         raise ValueError("4 waves, or 8 when the waves share the keys")
     if waves == 8 and head_dim > 160:
         raise ValueError("8 waves take head_dim up to 160 (wider heads would not fit the registers)")
+    if head_gate is not None and (head_gate.dtype != torch.float32 or head_gate.dim() != 2 or head_gate.stride(1) != 1
+                                  or head_gate.shape[0] != q.shape[0] or head_gate.shape[1] < n_heads):
+        raise ValueError("head_gate must be float32 [N, >= n_heads] with unit inner stride")
     if n_seqs == 0 or n_tokens == 0:
         return out
     ws_o = ws_ml = arrive = None
@@ -721,7 +743,11 @@ def attention_mfma(out: torch.Tensor, q: torch.Tensor, k_pool: torch.Tensor, v_p
         ws_o = torch.empty((q.shape[0] * n_heads * num_splits * head_dim,), dtype=torch.float32, device=dev)
         ws_ml = torch.empty((q.shape[0] * n_heads * num_splits * 2,), dtype=torch.float32, device=dev)
     scale = 1.0 / math.sqrt(head_dim) if scale is None else scale
-    _check(load("attention_mfma").llms_attention_mfma(
+    if head_gate is None:
+        entry, gate_args = load("attention_mfma").llms_attention_mfma, ()
+    else:
+        entry, gate_args = load("attention_gated").llms_attention_mfma_gated, (_ptr(head_gate), c_int(head_gate.stride(0)))
+    _check(entry(
         _ptr(out), c_int(out.stride(0)), _ptr(q), c_int(q.stride(0)), _ptr(k_pool), _ptr(v_pool),
         _ptr(block_tables), _ptr(table_rows), c_int(block_tables.shape[1]), _ptr(cu_seqlens), _ptr(context_lens),
         c_int(seq_begin),
@@ -729,7 +755,7 @@ def attention_mfma(out: torch.Tensor, q: torch.Tensor, k_pool: torch.Tensor, v_p
         c_int(head_dim), c_int(block_size), c_int(window), c_float(scale),
         c_int(1 if split_waves else 0),
         c_int(num_splits), c_int(waves), _ptr(ws_o), _ptr(ws_ml), _ptr(arrive),
-        c_int(arrive.numel() if arrive is not None else 0), _stream(dev)), "attention_mfma")
+        c_int(arrive.numel() if arrive is not None else 0), *gate_args, _stream(dev)), "attention_mfma")
     return out
 
 
@@ -999,20 +1025,22 @@ def conv_state(state: torch.Tensor, proj: torch.Tensor, state_slots: torch.Tenso
         "conv_state")
 
 
-def _check_dist_bias_and_gate(dist_bias, gate, heads: int, dv: int, n: int) -> None:
+def _check_dist_bias_and_gate(dist_bias, gate, heads: int, dv: int, n: int, gate_heads: bool = False) -> None:
     if dist_bias is not None and (dist_bias.dtype != torch.float32 or dist_bias.dim() != 2 or dist_bias.shape[0] != heads
                                   or dist_bias.shape[1] < 1 or not dist_bias.is_contiguous()):
         raise ValueError(f"dist_bias must be a contiguous float32 [{heads}, R + 1] tensor")
     if gate is not None and (gate.dtype != torch.float32 or gate.dim() != 2 or gate.stride(1) != 1 or gate.shape[0] != n
-                             or gate.shape[1] < heads * dv):
-        raise ValueError(f"gate must be float32 [{n}, >= {heads * dv}] with unit inner stride")
+                             or gate.shape[1] < (heads if gate_heads else heads * dv)):
+        raise ValueError(f"gate must be float32 [{n}, >= {heads if gate_heads else heads * dv}] with unit inner stride")
 
 
 def norm_store(q_out: torch.Tensor, proj: torch.Tensor, *, q_heads: int, k_heads: int, dk: int, v_heads: int, dv: int,
                q_norm: torch.Tensor | None = None, k_norm: torch.Tensor | None = None, eps: float = 0.0,
                temp_coef: float = 0.0, temp_every: int = 0, positions: torch.Tensor | None = None,
                slots: torch.Tensor | None = None, k_pool: torch.Tensor | None = None, v_pool: torch.Tensor | None = None,
-               block_size: int = 0, freq: torch.Tensor | None = None, unit_norm: bool = False) -> torch.Tensor:
+               block_size: int = 0, freq: torch.Tensor | None = None, unit_norm: bool = False,
+               angles: torch.Tensor | None = None, pairing: str = "half", norm_first: bool = False,
+               q_scale: torch.Tensor | None = None, values_from_keys: bool = False) -> torch.Tensor:
     """proj float32 [N, >= q_heads*dk + k_heads*dk + v_heads*dv] (q, k, v side by side; unit inner stride): with
     `freq` (float32 [rot_dims / 2]) the first rot_dims numbers of every head of q and k are first turned by the
     token's position (dimension i with dimension i + rot_dims / 2, angle position * freq[i]); `unit_norm`: every head
@@ -1020,9 +1048,21 @@ def norm_store(q_out: torch.Tensor, proj: torch.Tensor, *, q_heads: int, k_heads
     head of q and of k is divided by its root mean square (eps inside the root) and multiplied by `q_norm` / `k_norm`
     (float32 [dk], shared by the heads; None: the head passes as it is); q is multiplied by
     1 + temp_coef * ln(floor((p + 1) / temp_every) + 1) at position p (temp_every 0: no factor); rounded once: queries
-    to q_out [N, q_heads*dk], keys and values to the tokens' cache slots (`slots`; None: nothing is stored)."""
-    dev = _dev(q_out, proj, q_norm, k_norm, positions, slots, k_pool, v_pool, freq)
+    to q_out [N, q_heads*dk], keys and values to the tokens' cache slots (`slots`; None: nothing is stored).
+    `pairing` "neighbours": dimensions 2i and 2i + 1 turn together.  `norm_first`: the rotation comes behind the norm.
+    `angles` (rotary_angles(positions, freq), float32 [N, rot_dims / 2, 2]): the step's sines and cosines, which saves
+    working them out (the same to the bit).  `q_scale` float32 [q_heads]: a factor per query head.  `values_from_keys`:
+    proj holds no values; they are the keys as projected (v_heads = k_heads, dv = dk)."""
+    dev = _dev(q_out, proj, q_norm, k_norm, positions, slots, k_pool, v_pool, freq, angles, q_scale)
     n = proj.shape[0]
+    if values_from_keys and (v_heads != k_heads or dv != dk):
+        raise ValueError("values that are the keys have the keys' heads and size")
+    if angles is not None:
+        if freq is None:
+            raise ValueError("angles come with their frequencies")
+        _f32(angles, "angles", n * 2 * freq.numel())
+    if q_scale is not None:
+        _f32(q_scale, "q_scale", q_heads)
     rot_dims = 0
     if freq is not None:
         _f32(freq, "freq")
@@ -1030,7 +1070,7 @@ def norm_store(q_out: torch.Tensor, proj: torch.Tensor, *, q_heads: int, k_heads
         if rot_dims > dk:
             raise ValueError(f"{rot_dims} turned dimensions in a head of {dk}")
         _i32(positions, "positions", n)
-    channels = (q_heads + k_heads) * dk + v_heads * dv
+    channels = (q_heads + k_heads) * dk + (0 if values_from_keys else v_heads * dv)
     if proj.dim() != 2 or proj.dtype != torch.float32 or proj.stride(1) != 1 or proj.shape[1] < channels:
         raise ValueError(f"proj must be float32 [N, >= {channels}] with unit inner stride")
     _rows(q_out, "q_out", q_heads * dk)
@@ -1058,7 +1098,8 @@ def norm_store(q_out: torch.Tensor, proj: torch.Tensor, *, q_heads: int, k_heads
         c_int(_code(q_out)), _ptr(q_out), c_int(q_out.stride(0)), _ptr(proj), c_int(proj.stride(0)), _ptr(q_norm),
         _ptr(k_norm), c_float(eps), c_float(temp_coef), c_int(temp_every), _ptr(positions), _ptr(slots), _ptr(k_pool),
         _ptr(v_pool), c_int(n), c_int(q_heads), c_int(k_heads), c_int(dk), c_int(v_heads), c_int(dv), c_int(block_size),
-        _ptr(freq), c_int(rot_dims), c_int(1 if unit_norm else 0), _stream(dev)), "norm_store")
+        _ptr(freq), _ptr(angles), c_int(rot_dims), c_int(1 if unit_norm else 0), c_int(0 if _pairing(pairing) else 1),
+        c_int(1 if norm_first else 0), _ptr(q_scale), c_int(1 if values_from_keys else 0), _stream(dev)), "norm_store")
     return q_out
 
 
@@ -1079,7 +1120,7 @@ def attend_composed(out: torch.Tensor, q: torch.Tensor, k_pool: torch.Tensor, v_
                     talk: torch.Tensor | None = None, lam: float = 0.0, head_norm: bool = False, eps: float = 0.0,
                     out_scale: float = 1.0, table_rows: torch.Tensor | None = None,
                     context_lens: torch.Tensor | None = None, dist_bias: torch.Tensor | None = None,
-                    gate: torch.Tensor | None = None, sink: bool = False) -> torch.Tensor:
+                    gate: torch.Tensor | None = None, sink: bool = False, gate_heads: bool = False) -> torch.Tensor:
     """Attention of N new tokens over the paged cache, one workgroup per token (all its heads), float32 or bfloat16
     storage, 32-bit arithmetic.  q [N, heads*maps*dk] (head by head, a head's maps side by side); k_pool
     [pages, kv_heads*maps, block, dk]; v_pool [pages, kv_heads, dv, block]; out [N, heads*dv].  A query at
@@ -1089,11 +1130,11 @@ def attend_composed(out: torch.Tensor, q: torch.Tensor, k_pool: torch.Tensor, v_
     `head_norm`: each head's result is divided by its root mean square (eps inside the root) and multiplied by
     out_scale.  `context_lens` [B]: rows of a request of length 0 are padding and give zeros.  `dist_bias` float32
     [heads, R + 1]: dist_bias[h, min(i - j, R)] is added to the scores.  `gate` float32 [N, >= heads*dv] (unit inner
-    stride): the result is multiplied by sigmoid(gate).  `sink`: the softmax's denominator holds one more term,
+    stride): the result is multiplied by sigmoid(gate); with `gate_heads` it is [N, >= heads], one number per head.  `sink`: the softmax's denominator holds one more term,
     exp(0), a key of score zero without a value."""
     dev = _dev(out, q, k_pool, v_pool, block_tables, token_seq, positions, slopes, talk, table_rows, context_lens,
                dist_bias, gate)
-    _check_dist_bias_and_gate(dist_bias, gate, heads, dv, q.shape[0])
+    _check_dist_bias_and_gate(dist_bias, gate, heads, dv, q.shape[0], gate_heads)
     n = q.shape[0]
     if q.dim() != 2 or q.stride(1) != 1 or q.shape[1] < heads * maps * dk:
         raise ValueError("q must be [N, >= heads*maps*dk] with unit inner stride")
@@ -1132,7 +1173,7 @@ def attend_composed(out: torch.Tensor, q: torch.Tensor, k_pool: torch.Tensor, v_
         c_int(block_size), c_int(window), c_int(keep_first), c_int(chunk), c_float(scale), _ptr(slopes), _ptr(talk),
         c_float(lam), c_int(1 if head_norm else 0), c_float(eps), c_float(out_scale), _ptr(dist_bias),
         c_int(dist_bias.shape[1] - 1 if dist_bias is not None else 0), _ptr(gate),
-        c_int(gate.stride(0) if gate is not None else 0), c_int(1 if sink else 0), _stream(dev)),
+        c_int(gate.stride(0) if gate is not None else 0), c_int(1 if gate_heads else 0), c_int(1 if sink else 0), _stream(dev)),
         "attend_composed")
     return out
 
@@ -1163,7 +1204,7 @@ def attend_composed_mfma(out: torch.Tensor, q: torch.Tensor, k_pool: torch.Tenso
                          chunk: int = 0, slopes: torch.Tensor | None = None, talk: torch.Tensor | None = None,
                          lam: float = 0.0, head_norm: bool = False, eps: float = 0.0, out_scale: float = 1.0,
                          table_rows: torch.Tensor | None = None, shares: int = 1, dist_bias: torch.Tensor | None = None,
-                         gate: torch.Tensor | None = None, sink: bool = False) -> torch.Tensor:
+                         gate: torch.Tensor | None = None, sink: bool = False, gate_heads: bool = False) -> torch.Tensor:
     """`attend_composed` on the matrix cores (bfloat16) for requests [seq_begin, seq_begin + n_seqs) of a step: request
     b owns rows cu_seqlens[b] .. cu_seqlens[b+1] of q and out, brings at most `max_new` tokens and is context_lens[b]
     long after the step (0: padding, left alone).  Same arguments and arithmetic otherwise; the weights are rounded
@@ -1206,9 +1247,10 @@ def attend_composed_mfma(out: torch.Tensor, q: torch.Tensor, k_pool: torch.Tenso
                                   or dist_bias.shape[1] < 1 or not dist_bias.is_contiguous()):
         raise ValueError("dist_bias must be a contiguous float32 [heads, reach + 1] tensor")
     if gate is not None and (talk is not None or gate.dtype != torch.float32 or gate.dim() != 2 or gate.stride(1) != 1
-                             or gate.shape[0] != q.shape[0] or gate.shape[1] < heads * dv or gate.stride(0) % 4
-                             or gate.data_ptr() % 16):
-        raise ValueError("gate must be float32 [N, >= heads*dv] with unit inner stride and 16-byte aligned rows (and no mixed heads)")
+                             or gate.shape[0] != q.shape[0] or gate.shape[1] < (heads if gate_heads else heads * dv)
+                             or (not gate_heads and (gate.stride(0) % 4 or gate.data_ptr() % 16))):
+        raise ValueError("gate must be float32 [N, >= heads*dv] with unit inner stride and 16-byte aligned rows, or with "
+                         "gate_heads [N, >= heads] (and no mixed heads)")
     if n_seqs == 0 or max_new <= 0 or q.shape[0] == 0:
         return out
     ws_stats = ws_o = None
@@ -1225,8 +1267,8 @@ def attend_composed_mfma(out: torch.Tensor, q: torch.Tensor, k_pool: torch.Tenso
         c_int(block_size), c_int(window), c_int(keep_first), c_int(chunk), c_float(scale), _ptr(slopes), _ptr(talk),
         c_float(lam), c_int(1 if head_norm else 0), c_float(eps), c_float(out_scale), c_int(shares), _ptr(ws_stats),
         _ptr(ws_o), c_int(q.shape[0]), _ptr(dist_bias), c_int(dist_bias.shape[1] - 1 if dist_bias is not None else 0),
-        _ptr(gate), c_int(gate.stride(0) if gate is not None else 0), c_int(1 if sink else 0), _stream(dev)),
-        "attend_composed_mfma")
+        _ptr(gate), c_int(gate.stride(0) if gate is not None else 0), c_int(1 if gate_heads else 0), c_int(1 if sink else 0),
+        _stream(dev)), "attend_composed_mfma")
     return out
 
 
@@ -1325,7 +1367,9 @@ def _pairing(pairing: str) -> int:
     return 1 if pairing == "half" else 0
 
 
-def _latent_rotation(freq: torch.Tensor | None, dr: int) -> int:
+def _latent_rotation(freq: torch.Tensor | None, dr: int, angles: torch.Tensor | None = None, n: int = 0) -> int:
+    if angles is not None:
+        _f32(angles, "angles", n * 2 * (freq.numel() if freq is not None else 0))
     if freq is None:
         return 0
     _f32(freq, "freq")
@@ -1338,20 +1382,21 @@ def _latent_rotation(freq: torch.Tensor | None, dr: int) -> int:
 def latent_prepare(z: torch.Tensor, *, col_q: int, q_rank: int, col_c: int | None, r: int, dr: int, wq: torch.Tensor,
                    wc: torch.Tensor | None, freq: torch.Tensor | None, positions: torch.Tensor, eps: float,
                    cq: torch.Tensor, pool: torch.Tensor | None = None, slots: torch.Tensor | None = None,
-                   pairing: str = "neighbours") -> torch.Tensor:
+                   pairing: str = "neighbours", angles: torch.Tensor | None = None) -> torch.Tensor:
     """From the 32-bit input products z [N, columns]: cq [N, q_rank] = z[:, col_q:][:q_rank] over its root mean
     square times wq; with `col_c`, the cache rows pool[slots[n]] = [z_c over its root mean square times wc ; the dr
     columns behind it with their first 2 len(freq) dimensions turned by the token's position (pairs 2i, 2i+1; with
     `pairing` "half" pairs i, i + len(freq))].
-    pool [pages, 1, block, r + dr] in the dtype of cq."""
-    dev = _dev(z, wq, wc, freq, positions, cq, pool, slots)
+    pool [pages, 1, block, r + dr] in the dtype of cq.  `angles`: rotary_angles(positions, freq), which saves working
+    them out."""
+    dev = _dev(z, wq, wc, freq, positions, cq, pool, slots, angles)
     if z.dim() != 2 or z.dtype != torch.float32 or z.stride(1) != 1:
         raise ValueError("z must be a float32 matrix with unit inner stride")
     n = z.shape[0]
     _rows(cq, "cq", q_rank)
     _f32(wq, "wq", q_rank)
     _i32(positions, "positions", n)
-    dims = _latent_rotation(freq, dr)
+    dims = _latent_rotation(freq, dr, angles, n)
     if col_q < 0 or col_q + q_rank > z.shape[1]:
         raise ValueError("the query latent's columns lie outside z")
     if col_c is not None:
@@ -1367,17 +1412,18 @@ def latent_prepare(z: torch.Tensor, *, col_q: int, q_rank: int, col_c: int | Non
         return cq
     _check(load("latent").llms_latent_prepare(
         c_int(_code(cq)), _ptr(cq), _ptr(pool if col_c is not None else None), _ptr(z), c_int(z.stride(0)), c_int(col_q),
-        c_int(q_rank), c_int(-1 if col_c is None else col_c), c_int(r), c_int(dr), _ptr(wq), _ptr(wc), _ptr(freq), c_int(dims),
+        c_int(q_rank), c_int(-1 if col_c is None else col_c), c_int(r), c_int(dr), _ptr(wq), _ptr(wc), _ptr(freq), _ptr(angles), c_int(dims),
         _ptr(positions), _ptr(slots if col_c is not None else None), c_float(eps), c_int(n), c_int(_pairing(pairing)),
         _stream(dev)), "latent_prepare")
     return cq
 
 
 def latent_query(plain: torch.Tensor, folded: torch.Tensor, q: torch.Tensor, *, heads: int, dn: int, dr: int, r: int,
-                 freq: torch.Tensor | None, positions: torch.Tensor, pairing: str = "neighbours") -> None:
+                 freq: torch.Tensor | None, positions: torch.Tensor, pairing: str = "neighbours",
+                 angles: torch.Tensor | None = None) -> None:
     """q [N, heads * (dn + dr)] float32 -> plain [N, heads * dn] (the unrotated parts) and folded[n, h, r:] (the
-    rotated parts, turned); folded [N, heads * (r + dr)]."""
-    dev = _dev(plain, folded, q, freq, positions)
+    rotated parts, turned); folded [N, heads * (r + dr)].  `angles` as in `latent_prepare`."""
+    dev = _dev(plain, folded, q, freq, positions, angles)
     n = q.shape[0]
     _f32(q, "q", n * heads * (dn + dr))
     _rows(plain, "plain", heads * dn)
@@ -1385,12 +1431,47 @@ def latent_query(plain: torch.Tensor, folded: torch.Tensor, q: torch.Tensor, *, 
     _i32(positions, "positions", n)
     if plain.dtype != folded.dtype or plain.shape[0] != n or folded.shape[0] != n:
         raise ValueError("plain and folded share one dtype and q's rows")
-    dims = _latent_rotation(freq, dr)
+    dims = _latent_rotation(freq, dr, angles, n)
     if n == 0:
         return
     _check(load("latent").llms_latent_query(
         c_int(_code(plain)), _ptr(plain), _ptr(folded), _ptr(q), c_int(heads), c_int(dn), c_int(dr), c_int(r), _ptr(freq),
-        c_int(dims), _ptr(positions), c_int(n), c_int(_pairing(pairing)), _stream(dev)), "latent_query")
+        _ptr(angles), c_int(dims), _ptr(positions), c_int(n), c_int(_pairing(pairing)), _stream(dev)), "latent_query")
+
+
+def latent_split(plain: torch.Tensor, folded: torch.Tensor, z: torch.Tensor, *, col_q: int, col_c: int | None, heads: int, dn: int,
+                 dr: int, r: int, wc: torch.Tensor | None, freq: torch.Tensor | None, positions: torch.Tensor, eps: float,
+                 pool: torch.Tensor | None = None, slots: torch.Tensor | None = None, pairing: str = "neighbours",
+                 angles: torch.Tensor | None = None) -> None:
+    """`latent_query` and the cache rows of `latent_prepare` in one launch, for queries that lie in z [N, columns] themselves
+    (heads * (dn + dr) columns from col_q on) instead of behind a latent of their own."""
+    dev = _dev(plain, folded, z, wc, freq, positions, pool, slots, angles)
+    if z.dim() != 2 or z.dtype != torch.float32 or z.stride(1) != 1:
+        raise ValueError("z must be a float32 matrix with unit inner stride")
+    n = z.shape[0]
+    _rows(plain, "plain", heads * dn)
+    _rows(folded, "folded", heads * (r + dr))
+    _i32(positions, "positions", n)
+    if plain.dtype != folded.dtype or plain.shape[0] != n or folded.shape[0] != n:
+        raise ValueError("plain and folded share one dtype and z's rows")
+    dims = _latent_rotation(freq, dr, angles, n)
+    if col_q < 0 or col_q + heads * (dn + dr) > z.shape[1]:
+        raise ValueError("the queries' columns lie outside z")
+    if col_c is not None:
+        if col_c < 0 or col_c + r + dr > z.shape[1]:
+            raise ValueError("the latent's columns lie outside z")
+        _f32(wc, "wc", r)
+        if pool is None or slots is None or pool.dtype != plain.dtype or not pool.is_contiguous() or pool.shape[-1] != r + dr:
+            raise ValueError("a layer that keeps a latent needs its pool [.., r + dr] in plain's dtype and the tokens' slots")
+        _i32(slots, "slots", n)
+    if n == 0:
+        return
+    keeps = col_c is not None
+    _check(load("latent").llms_latent_split(
+        c_int(_code(plain)), _ptr(plain), _ptr(folded), _ptr(pool if keeps else None), _ptr(z), c_int(z.stride(0)), c_int(col_q),
+        c_int(col_c if keeps else -1), c_int(heads), c_int(dn), c_int(dr), c_int(r), _ptr(wc if keeps else None), _ptr(freq),
+        _ptr(angles), c_int(dims), _ptr(positions), _ptr(slots if keeps else None), c_float(eps), c_int(n),
+        c_int(_pairing(pairing)), _stream(dev)), "latent_split")
 
 
 LATENT_ROW_MAX = 1024
@@ -1398,11 +1479,14 @@ LATENT_ROW_MAX = 1024
 
 def attend_latent(out: torch.Tensor, q: torch.Tensor, pool: torch.Tensor, block_tables: torch.Tensor,
                   token_seq: torch.Tensor, positions: torch.Tensor, context_lens: torch.Tensor, *, heads: int, r: int,
-                  dr: int, block_size: int, window: int, scale: float, table_rows: torch.Tensor | None = None) -> torch.Tensor:
+                  dr: int, block_size: int, window: int, scale: float, table_rows: torch.Tensor | None = None,
+                  sink: torch.Tensor | None = None) -> torch.Tensor:
     """out[n, h] = sum_j softmax_j(scale q[n, h] . row_j) row_j[:r] over the cache rows j of token n's request with
     0 <= position - j < window (window 0: every j <= position); q [N, heads * (r + dr)], out [N, heads * r], pool
-    [pages, 1, block, r + dr]."""
-    dev = _dev(out, q, pool, block_tables, token_seq, positions, context_lens, table_rows)
+    [pages, 1, block, r + dr].  `sink` float32 [heads]: head h's denominator holds one more term, exp(sink[h])."""
+    dev = _dev(out, q, pool, block_tables, token_seq, positions, context_lens, table_rows, sink)
+    if sink is not None:
+        _f32(sink, "sink", heads)
     n = q.shape[0]
     _rows(q, "q", heads * (r + dr))
     _rows(out, "out", heads * r)
@@ -1428,7 +1512,7 @@ def attend_latent(out: torch.Tensor, q: torch.Tensor, pool: torch.Tensor, block_
     _check(load("latent").llms_attend_latent(
         c_int(_code(q)), _ptr(out), _ptr(q), _ptr(pool), _ptr(block_tables), c_int(block_tables.shape[1]), _ptr(table_rows),
         _ptr(token_seq), _ptr(positions), _ptr(context_lens), c_int(n), c_int(heads), c_int(r), c_int(dr), c_int(block_size),
-        c_int(window), c_float(scale), _stream(dev)), "attend_latent")
+        c_int(window), c_float(scale), _ptr(sink), _stream(dev)), "attend_latent")
     return out
 
 
@@ -1449,11 +1533,13 @@ def attend_latent_mfma_supported(dtype: torch.dtype, r: int, dr: int) -> bool:
 def attend_latent_mfma(out: torch.Tensor, q: torch.Tensor, pool: torch.Tensor, block_tables: torch.Tensor,
                        cu_seqlens: torch.Tensor, context_lens: torch.Tensor, *, n_seqs: int, max_count: int, heads: int,
                        r: int, dr: int, block_size: int, window: int, scale: float, splits: int = 1,
-                       table_rows: torch.Tensor | None = None) -> torch.Tensor:
+                       table_rows: torch.Tensor | None = None, sink: torch.Tensor | None = None) -> torch.Tensor:
     """`attend_latent` on the matrix cores for the requests [0, n_seqs) of a step: request b owns the rows
     cu_seqlens[b] .. cu_seqlens[b + 1] of q and out, which are its last tokens (positions context_lens[b] - count ..).
     `max_count`: no request brings more rows.  `splits`: workgroups that share the keys of one block of rows."""
-    dev = _dev(out, q, pool, block_tables, cu_seqlens, context_lens, table_rows)
+    dev = _dev(out, q, pool, block_tables, cu_seqlens, context_lens, table_rows, sink)
+    if sink is not None:
+        _f32(sink, "sink", heads)
     n = q.shape[0]
     _rows(q, "q", heads * (r + dr))
     _rows(out, "out", heads * r)
@@ -1483,7 +1569,7 @@ def attend_latent_mfma(out: torch.Tensor, q: torch.Tensor, pool: torch.Tensor, b
     _check(load("latent_mfma").llms_attend_latent_mfma(
         _ptr(out), _ptr(q), _ptr(pool), _ptr(block_tables), c_int(block_tables.shape[1]), _ptr(table_rows), _ptr(cu_seqlens),
         _ptr(context_lens), _ptr(ws), c_int(n_seqs), c_int(n), c_int(max_count), c_int(heads), c_int(r), c_int(dr),
-        c_int(block_size), c_int(window), c_float(scale), c_int(splits), _stream(dev)), "attend_latent_mfma")
+        c_int(block_size), c_int(window), c_float(scale), c_int(splits), _ptr(sink), _stream(dev)), "attend_latent_mfma")
     return out
 
 
@@ -1520,7 +1606,7 @@ def _grouped_on_matrix_cores(x: torch.Tensor, w: torch.Tensor, x_ld: int, x_gs: 
 def grouped_product(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor, *, epilogue: str = "plain",
                     segments: "tuple[torch.Tensor, torch.Tensor] | None" = None, gate: torch.Tensor | None = None,
                     gate_column: int = 0, limit: float = 0.0, units: int = 0, k_parts: int = 1,
-                    unit: str = "clamped") -> torch.Tensor:
+                    unit: str = "clamped", gate_per_group: bool = False) -> torch.Tensor:
     """w [G, N, K].  Without `segments` every row meets every group: x [M, G, K] and out [M, G, N'] (views whose
     last axis has unit stride; the strides of the other two are free), out[m, g] = x[m, g] w[g]^T.  With `segments`
     = (seg [G + 1], tile_start [2, G + 1]) on the device (what `moe_sort` returns), x [M, K] and out [M, N'] hold rows
@@ -1528,7 +1614,7 @@ def grouped_product(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor, *, epil
     Epilogues: "plain" (N' = N); "paired" (N' = `units`: w is `stack_paired(a, b)`,
     out = min(a, limit) sigmoid(1.702 min(a, limit)) (clamp(b, +-limit) + 1), or with `unit` "silu"
     out = a sigmoid(a) b); "gated" (out times
-    sigmoid(gate[m, gate_column + g N + n]), gate float32 [M, columns]).
+    sigmoid(gate[m, gate_column + g N + n]), gate float32 [M, columns]; `gate_per_group`: sigmoid(gate[m, gate_column + g])).
     bfloat16 operands with K and the strides of x in multiples of 8 go to the matrix cores, all else to the 32-bit
     multiply-add kernel.  `k_parts` > 1 (as `grouped_k_parts` allows): out is float32 [k_parts, M, N] and holds partial
     sums over shares of K, for the caller to add up."""
@@ -1577,19 +1663,19 @@ def grouped_product(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor, *, epil
         tile = GROUPED_TILE_MFMA if mfma else GROUPED_TILE
         seg_ptr, tiles_ptr = seg, tiles.view(2, g + 1)[1 if mfma else 0]
         max_tiles = -(-m // tile) + g
-    z_ld = z_gs = 0
+    z_ld = z_gs = z_ns = 0
     z = None
     if epilogue == "gated":
         if gate is None or gate.dtype != torch.float32 or gate.dim() != 2 or gate.stride(1) != 1 or gate.shape[0] != m:
             raise ValueError("the gated epilogue needs float32 gate products [M, columns]")
-        if gate_column < 0 or gate_column + g * n > gate.shape[1]:
+        if gate_column < 0 or gate_column + (g if gate_per_group else g * n) > gate.shape[1]:
             raise ValueError("the gate's columns lie outside the gate products")
-        z, z_ld, z_gs = gate[:, gate_column:], gate.stride(0), n
+        z, z_ld, z_gs, z_ns = gate[:, gate_column:], gate.stride(0), 1 if gate_per_group else n, 0 if gate_per_group else 1
     if m == 0:
         return out
     common = (_ptr(out), c_long(out_ld), c_long(out_gs), _ptr(x), c_long(x_ld), c_long(x_gs), _ptr(w), c_int(m), c_int(n),
               c_int(k), c_int(g), _ptr(seg_ptr), _ptr(tiles_ptr), c_int(max_tiles), _ptr(z), c_long(z_ld), c_long(z_gs),
-              c_float(limit), c_int(_GATED_UNITS[unit]), c_int(units), _stream(dev))
+              c_int(z_ns), c_float(limit), c_int(_GATED_UNITS[unit]), c_int(units), _stream(dev))
     lib = load("grouped_gemm")
     if mfma:
         _check(lib.llms_grouped_mfma(c_int(_code(out)), c_int(_EPILOGUES[epilogue]), *common[:-1], c_int(k_parts),
@@ -1617,14 +1703,16 @@ MOE_MAX_TOP = 16
 
 def moe_router(chosen: torch.Tensor, weight: torch.Tensor, h: torch.Tensor, w_router: torch.Tensor, *,
                renormalize: bool = False, scores: str = "sigmoid", groups: int = 1, keep: int = 1,
-               renorm_eps: float = 0.0, bias: torch.Tensor | None = None, extra_out: torch.Tensor | None = None) -> None:
+               renorm_eps: float = 0.0, bias: torch.Tensor | None = None, extra_out: torch.Tensor | None = None,
+               correction: torch.Tensor | None = None, scale: float = 1.0) -> None:
     """Per row of h [N, hidden]: scores sigmoid(W_router h), or with `scores` "softmax" the softmax over all experts,
     in 32-bit; the `top` largest in descending order (the lower expert wins a tie) into chosen int32 [N, top], their
     scores (over their sum + `renorm_eps` with `renormalize`) into weight float32 [N, top].  `groups` > 1: the experts
     form that many equal groups of neighbours, a group's score is its largest, and only experts of the `keep` best
-    groups can be chosen.  `bias` float32 [experts] is added to z.  `extra_out` float32 [N, extra]: w_router holds
+    groups can be chosen.  `correction` float32 [experts]: the choice (groups included) is made on score + correction, the
+    weights stay the scores.  Every weight is multiplied by `scale`.  `bias` float32 [experts] is added to z.  `extra_out` float32 [N, extra]: w_router holds
     `extra` more rows behind the experts', whose products with h are stored there as they are."""
-    dev = _dev(chosen, weight, h, w_router, bias, extra_out)
+    dev = _dev(chosen, weight, h, w_router, bias, extra_out, correction)
     _rows(h, "h")
     _rows(w_router, "w_router", h.shape[1])
     n, top = h.shape[0], chosen.shape[-1]
@@ -1641,6 +1729,8 @@ def moe_router(chosen: torch.Tensor, weight: torch.Tensor, h: torch.Tensor, w_ro
         raise ValueError("w_router holds no experts' rows")
     if bias is not None:
         _f32(bias, "bias", experts)
+    if correction is not None:
+        _f32(correction, "correction", experts)
     if h.dtype != w_router.dtype:
         raise ValueError("h and w_router differ in dtype")
     if not 1 <= top <= min(MOE_MAX_TOP, experts):
@@ -1654,7 +1744,8 @@ def moe_router(chosen: torch.Tensor, weight: torch.Tensor, h: torch.Tensor, w_ro
     _check(load("moe").llms_moe_router(
         c_int(_code(h)), _ptr(chosen), _ptr(weight), _ptr(h), _ptr(w_router), c_int(n), c_int(h.shape[1]), c_int(experts),
         c_int(top), c_int(1 if renormalize else 0), c_int(1 if scores == "softmax" else 0), c_int(groups), c_int(keep),
-        c_float(renorm_eps), _ptr(bias), c_int(extra), _ptr(extra_out), _stream(dev)), "moe_router")
+        c_float(renorm_eps), _ptr(bias), c_int(extra), _ptr(extra_out), _ptr(correction), c_float(scale),
+        _stream(dev)), "moe_router")
 
 
 def moe_sort(chosen: torch.Tensor, experts: int):

@@ -151,44 +151,54 @@ class Attention(Mixer):
                                table_rows=batch.state_slots)
 
     def prompt_splits(self, n_requests: int, max_new: int, max_context: int, cus: int = 256) -> int:
-        """Workgroups that share the keys of one block of prompt tokens (a second kernel merges their shares).
-        Blocks enough for a workgroup of 8 waves on every CU need no sharing: there each wave has a twin that
-        takes every other tile of keys for the same tokens, and with two such workgroups per CU the long blocks
-        and the short ones even out.  With exactly one per CU sharing pays only behind a long prefix (measured:
-        from about 3,000 keys on).  A short portion behind a long prefix has few blocks and many keys: its keys
-        are shared out, 8 tiles of keys a workgroup at least (16 where the blocks alone are half a chip), up to
-        about two workgroups of 4 waves per CU, and not in more than 4 once the blocks alone are a quarter of a
-        chip (measured on portions of 16 to 256 tokens behind 256 to 4,032 keys, at head sizes 64 and 128: the
-        merge kernel's work grows with blocks times shares).  `cus`: the device's compute units."""
-        if self.window:
-            return 1
-        g = self.num_heads // self.num_kv_heads
-        hg = min(g, 16)
-        blocks = -(-max_new // (4 * (16 // hg)))  # of 4 waves with one column group each
-        workgroups = blocks * self.num_kv_heads * -(-g // hg) * n_requests
-        tiles = -(-max_context // 32)
-        if workgroups >= 2 * cus:
-            return 1
-        if workgroups >= cus:
-            return 4 if tiles >= 96 else 1
-        per_share = 16 if workgroups >= cus // 2 else 8
-        most = 4 if workgroups >= cus // 4 else 8
-        return max(1, min(2 * cus // max(workgroups, 1), tiles // per_share, most))
+        return prompt_splits(self.num_heads, self.num_kv_heads, self.window, n_requests, max_new, max_context, cus)
 
     def decode_arrangement(self, n_requests: int, max_context: int, cus: int = 256) -> tuple[int, int]:
-        """(workgroups per request and KV head, waves per workgroup) for decoding.  The waves of a
-        workgroup take 32 keys at a time each and merge in LDS; workgroups that share a request hand
-        their shares to the one that finishes last, through memory, which costs more (2 to 3
-        microseconds) than a few extra tiles per wave.  So a small batch first gets 8 waves, and is
-        split over workgroups only when a wave would still walk more than 4 tiles (measured: at a
-        context of 512 no split pays at any batch size, at 4,096 four to eight do up to batch 8); once
-        the batch alone fills the chip (a workgroup for each of its `cus` compute units) nothing is split."""
-        g = self.num_heads // self.num_kv_heads
-        groups = n_requests * self.num_kv_heads * -(-g // 16)
-        reach = min(max_context, self.window) if self.window else max_context
-        waves = 8 if self.head_dim <= 160 else 4  # (8 waves of wider heads would not fit the registers)
-        if groups >= cus:
-            return 1, waves
-        tiles = -(-reach // 32)
-        splits = max(1, min(cus // groups, -(-tiles // (4 * waves))))
-        return splits, waves
+        return decode_arrangement(self.num_heads, self.num_kv_heads, self.head_dim, self.window, n_requests, max_context, cus)
+
+
+def prompt_splits(num_heads: int, num_kv_heads: int, window: int | None, n_requests: int, max_new: int,
+                  max_context: int, cus: int = 256) -> int:
+    """Workgroups that share the keys of one block of prompt tokens (a second kernel merges their shares).
+    Blocks enough for a workgroup of 8 waves on every CU need no sharing: there each wave has a twin that
+    takes every other tile of keys for the same tokens, and with two such workgroups per CU the long blocks
+    and the short ones even out.  With exactly one per CU sharing pays only behind a long prefix (measured:
+    from about 3,000 keys on).  A short portion behind a long prefix has few blocks and many keys: its keys
+    are shared out, 8 tiles of keys a workgroup at least (16 where the blocks alone are half a chip), up to
+    about two workgroups of 4 waves per CU, and not in more than 4 once the blocks alone are a quarter of a
+    chip (measured on portions of 16 to 256 tokens behind 256 to 4,032 keys, at head sizes 64 and 128: the
+    merge kernel's work grows with blocks times shares).  `cus`: the device's compute units."""
+    if window:
+        return 1
+    g = num_heads // num_kv_heads
+    hg = min(g, 16)
+    blocks = -(-max_new // (4 * (16 // hg)))  # of 4 waves with one column group each
+    workgroups = blocks * num_kv_heads * -(-g // hg) * n_requests
+    tiles = -(-max_context // 32)
+    if workgroups >= 2 * cus:
+        return 1
+    if workgroups >= cus:
+        return 4 if tiles >= 96 else 1
+    per_share = 16 if workgroups >= cus // 2 else 8
+    most = 4 if workgroups >= cus // 4 else 8
+    return max(1, min(2 * cus // max(workgroups, 1), tiles // per_share, most))
+
+
+def decode_arrangement(num_heads: int, num_kv_heads: int, head_dim: int, window: int | None, n_requests: int, max_context: int,
+                       cus: int = 256) -> tuple[int, int]:
+    """(workgroups per request and KV head, waves per workgroup) for decoding.  The waves of a
+    workgroup take 32 keys at a time each and merge in LDS; workgroups that share a request hand
+    their shares to the one that finishes last, through memory, which costs more (2 to 3
+    microseconds) than a few extra tiles per wave.  So a small batch first gets 8 waves, and is
+    split over workgroups only when a wave would still walk more than 4 tiles (measured: at a
+    context of 512 no split pays at any batch size, at 4,096 four to eight do up to batch 8); once
+    the batch alone fills the chip (a workgroup for each of its `cus` compute units) nothing is split."""
+    g = num_heads // num_kv_heads
+    groups = n_requests * num_kv_heads * -(-g // 16)
+    reach = min(max_context, window) if window else max_context
+    waves = 8 if head_dim <= 160 else 4  # (8 waves of wider heads would not fit the registers)
+    if groups >= cus:
+        return 1, waves
+    tiles = -(-reach // 32)
+    splits = max(1, min(cus // groups, -(-tiles // (4 * waves))))
+    return splits, waves

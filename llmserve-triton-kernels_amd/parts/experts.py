@@ -7,8 +7,10 @@ out: scores ("sigmoid" or "softmax" over all experts), groups and keep (the expe
 neighbours, a group's score is its largest, only experts of the `keep` best groups can be chosen), renorm_eps (added
 to the sum that `renormalize` divides by), weight_on ("input": the weight multiplies the expert's input; "output":
 its result), unit ("clamped" or "silu"), router_bias (True: a bias per expert, tensor "<router>.b", is added to z),
-shared ({"intermediate": I, "gate": True or False}: one more SiLU-gated unit of its own width that every token uses,
-tensors "shared.gate", "shared.up", "shared.down"; with "gate" its result is multiplied by sigmoid(w_sg . h), one number
+correction (True: a number per expert, tensor "correction", is added to the scores for the choice only), weight_scale (the
+weights are multiplied by it; default 1),
+shared ({"intermediate": I, "gate": True or False, "unit": "silu" (default) or "clamped" with "limit"}: one more gated unit
+of its own width that every token uses, tensors "shared.gate", "shared.up", "shared.down"; with "gate" its result is multiplied by sigmoid(w_sg . h), one number
 per token, tensor "shared.sg" [1, hidden]).
 
 Router: z = W_router h in 32-bit, scores sigmoid(z) or softmax(z), the `top` largest chosen.  With weight_on
@@ -32,7 +34,8 @@ from .registry import FeedForward, register_feed_forward
 from .spec import ParamInfo
 
 _DEFAULT_NAMES = {"router": "router", "gate": "e{e}.gate", "up": "e{e}.up", "down": "e{e}.down", "router_bias": "router.b",
-                  "shared_gate": "shared.gate", "shared_up": "shared.up", "shared_down": "shared.down", "shared_sg": "shared.sg"}
+                  "shared_gate": "shared.gate", "shared_up": "shared.up", "shared_down": "shared.down", "shared_sg": "shared.sg",
+                  "correction": "correction"}
 
 
 @register_feed_forward("experts")
@@ -62,6 +65,9 @@ class Experts(FeedForward):
                              f"of which {self.top} are chosen")
         self.names = dict(_DEFAULT_NAMES, **(spec.get("names") or {}))
         self.router_bias = bool(spec.get("router_bias", False))
+        self.correction = bool(spec.get("correction", False))
+        self.weight_scale = float(spec.get("weight_scale", 1.0))
+        self.w_correction = None
         shared = spec.get("shared") or None
         self.shared_intermediate = int(shared["intermediate"]) if shared else 0
         self.shared_gated = bool(shared.get("gate", False)) if shared else False
@@ -76,6 +82,7 @@ class Experts(FeedForward):
             n = self.names
             self.shared_unit = FEED_FORWARDS.build(PartSpec("swiglu", {
                 "hidden": self.hidden, "intermediate": self.shared_intermediate, "result": "float32",
+                "unit": shared.get("unit", "silu"), "limit": shared.get("limit", 0.0),
                 "names": {"gate": n["shared_gate"], "up": n["shared_up"], "down": n["shared_down"]}}), ctx)
         if not 1 <= self.top <= min(self.experts, ops.MOE_MAX_TOP):
             raise ValueError(f"top={self.top} of {self.experts} experts (at most {ops.MOE_MAX_TOP})")
@@ -93,6 +100,8 @@ class Experts(FeedForward):
             infos[n["down"].format(e=e)] = ParamInfo((h, i))
         if self.router_bias:
             infos[n["router_bias"]] = ParamInfo((self.experts,), "around_zero")
+        if self.correction:
+            infos[n["correction"]] = ParamInfo((self.experts,), "around_zero")
         if self.shared_unit is not None:
             infos.update(self.shared_unit.param_infos())
             if self.shared_gated:
@@ -104,6 +113,8 @@ class Experts(FeedForward):
         self.w_router = tensors[n["router"]].contiguous()
         if self.router_bias:
             self.b_router = tensors[n["router_bias"]].float().contiguous()
+        if self.correction:
+            self.w_correction = tensors[n["correction"]].float().contiguous()
         if self.shared_unit is not None:
             self.shared_unit.load({name: tensors[name] for name in self.shared_unit.param_infos()})
             if self.shared_gated:  # the gate's row lies behind the experts' in the router's matrix: one kernel forms both
@@ -122,7 +133,7 @@ class Experts(FeedForward):
         shared_gate = torch.empty((rows, 1), dtype=torch.float32, device=dev) if self.shared_gated else None
         ops.moe_router(chosen, weight, x, self.w_router, renormalize=self.renormalize, scores=self.scores,
                        groups=self.groups, keep=self.keep, renorm_eps=self.renorm_eps, bias=self.b_router,
-                       extra_out=shared_gate)
+                       extra_out=shared_gate, correction=self.w_correction, scale=self.weight_scale)
         shared = self.shared_unit.forward(x) if self.shared_unit is not None else None
         on_input = self.weight_on == "input"
         sorted_in = torch.empty((pairs, self.hidden), dtype=x.dtype, device=dev)

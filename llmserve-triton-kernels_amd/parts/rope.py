@@ -15,6 +15,19 @@ from ..ops import library as ops
 from .registry import PositionEncoding, register_position_encoding
 
 
+def step_angles(batch, freq, key) -> "torch.Tensor | None":
+    """float32 [N, len(freq), 2]: sine and cosine of every new token's position times every frequency (None: nothing
+    turns).  Worked out by the first part of a step that asks; the others whose frequencies go by the same `key` find the
+    table in what the step's parts share."""
+    shared = getattr(batch, "shared", None)
+    if freq is None or shared is None:
+        return None
+    key = ("step_angles", key)
+    if key not in shared:
+        shared[key] = ops.rotary_angles(batch.positions, freq)
+    return shared[key]
+
+
 @register_position_encoding("rope")
 class RotaryEncoding(PositionEncoding):
     graph_safe = True

@@ -1,5 +1,6 @@
 """Gated feed-forward: down(silu(gate(x)) * up(x)), no biases
-(src/llmserve/model/llama.py:112-120).  Parameters: hidden, intermediate.
+(src/llmserve/model/llama.py:112-120).  Parameters: hidden, intermediate, and optionally unit ("silu", or "clamped" with
+`limit`: down(g sigmoid(1.702 g) (u + 1)), g = min(gate(x), limit), u = clamp(up(x), -limit, limit)).
 gate_proj and up_proj are stacked into one [2I, H] matrix at load, so one product feeds
 the activation.  With few bfloat16 rows that product also does the activation after it
 (ops.gemm_stream); otherwise the product and the activation are kernels of their own."""
@@ -28,6 +29,10 @@ class SwiGLU(FeedForward):
         names = spec.get("names") or {}
         self.names = {k: names.get(k, f"{k}_proj.weight") for k in ("gate", "up", "down")}
         self.result_dtype = torch.float32 if spec.get("result", "model") == "float32" else None
+        self.unit = spec.get("unit", "silu")
+        if self.unit not in ("silu", "clamped"):
+            raise ValueError(f"unit={self.unit!r}; choose 'silu' or 'clamped'")
+        self.limit = float(spec["limit"]) if self.unit == "clamped" else None
         self.gate_up: torch.Tensor | None = None
         self.down: torch.Tensor | None = None
 
@@ -52,15 +57,15 @@ class SwiGLU(FeedForward):
                 x.resolve(None)  # nothing is left to add: the kernel norms the residual rows as they are
             elif deferred:
                 rows = x.materialize()
-            ops.gemm_decode(act, rows, self.gate_up, swiglu=True, norm=norm)  # norm before, activation after the product
+            ops.gemm_decode(act, rows, self.gate_up, swiglu=True, norm=norm, limit=self.limit)  # norm before, activation after the product
         else:
             if deferred:
                 rows = x.materialize()
             few = dtype == torch.bfloat16 and few_rows(m, self.gate_up) and self.intermediate % 8 == 0
             if few and ops.gemm_bf16_supported(rows, self.gate_up):
-                ops.gemm_stream(act, rows, self.gate_up, swiglu=True)  # activation in the product's epilogue
+                ops.gemm_stream(act, rows, self.gate_up, swiglu=True, limit=self.limit)  # activation in the product's epilogue
             else:
-                ops.silu_mul(act, linear(rows, self.gate_up))
+                ops.silu_mul(act, linear(rows, self.gate_up), self.limit)
         if deferred and x.may_add_in_place and adds_residual_in_epilogue(act, self.down):
             ops.gemm_decode(None, act, self.down, residual=x.residual)  # the residual sum in the product's epilogue
             return ADDED_IN_PLACE
