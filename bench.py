@@ -26,12 +26,13 @@ first token, inter-token latency percentiles and the number of preemptions besid
 `--pages-fraction` shrinks the cache pool below what the whole workload needs, so that
 requests wait and are preempted.
 
-    python bench.py --workload designs [--design dibepel|milozen|felavik|nolavik] [--beside llama|felavik|...] [--sizes 1b,7b] [--layers 6] [--batches 8,32] [--context 512]
+    python bench.py --workload designs [--design dibepel|milozen|felavik|nolavik|zotunex] [--beside llama|felavik|...] [--sizes 1b,7b] [--layers 6] [--batches 8,32] [--context 512]
 
 puts the Dibepel design (or, with `--design milozen`, the Milozen design: latent attention, experts, two streams; with
 `--design felavik`, the Felavik design: linear attention with a decay per head, gated softmax attention, experts in groups;
 with `--design nolavik`, the Nolavik design: latent attention, the gated delta rule, sink attention beside a selective scan,
-experts with a shared expert, a looped layer)
+experts with a shared expert, a looped layer; with `--design zotunex`, the Zotunex design: attention whose values are its
+keys, latent attention with sinks, squared-relu and expert feed-forwards)
 beside the Llama decoder at equal layer sizes (width, heads, key/value heads, head size,
 feed-forward, vocabulary, layers; random weights): prefill tokens a second for one prompt of 2,048 tokens in one
 step, and decoded tokens a second at the given batch sizes behind `--context` tokens, both through the step
@@ -296,6 +297,31 @@ def nolavik_config(size: dict, layers: int, experts: int = 8, top: int = 2) -> d
             "loop": {"start": 1, "stop": 2, "times": 2 if layers > 2 else 1}}
 
 
+def zotunex_config(size: dict, layers: int, experts: int = 8, top: int = 2) -> dict:
+    """Every third layer, from the second, latent attention (as many heads as the Llama shape, the head size unrotated and half
+    of it rotated, a latent of four head sizes); the others softmax attention of the Llama shape's heads and key/value heads
+    whose values are the keys (half of every head turned, frequencies divided by 8).  The first layer's feed-forward is the
+    squared relu between two matrices of one and a half times the dense width (the weights of the gated one); the others
+    choose `top` of `experts` experts of a quarter of the dense width and have a shared expert of half of it."""
+    dim, heads, width = size["dim"], size["heads"], size["width"]
+    mlp = {"kind": "moe", "expert": {"ff": size["ff"] // 4, "limit": 7.0}, "router": {"experts": experts, "top": top, "scale": 2.0},
+           "shared": {"ff": size["ff"] // 2, "limit": 7.0}}
+    entries = []
+    for i in range(layers):
+        if i % 3 == 1:
+            entry = {"type": "latent_attention", "mixer": {
+                "heads": heads, "dim": dim, "rot_dim": dim // 2, "vdim": dim, "kv_rank": 4 * dim, "scale": (dim + dim // 2) ** -0.5,
+                "rot": {"base": 1000000.0, "dims": dim // 2}}}
+        else:
+            entry = {"type": "attention", "mixer": {
+                "heads": heads, "kv_heads": size["kv_heads"], "dim": dim, "vdim": dim, "scale": dim ** -0.5,
+                "rot": {"base": 10000.0, "dims": dim // 2, "scaling": {"factor": 8.0}}}}
+        entry["mlp"] = {"kind": "dense", "ff": size["ff"] * 3 // 2} if i == 0 else mlp
+        entries.append(entry)
+    return {"architecture": "Zotunex", "vocab": size["vocab"], "width": width, "embedding": {"scale": 8.0}, "norm": {"eps": 1e-6},
+            "layers": entries}
+
+
 def llama_config(size: dict, layers: int, positions: int) -> dict:
     return dict(architectures=["LlamaForCausalLM"], model_type="llama", vocab_size=size["vocab"], hidden_size=size["width"],
                 intermediate_size=size["ff"], num_hidden_layers=layers, num_attention_heads=size["heads"],
@@ -370,7 +396,8 @@ def designs(args) -> int:
 
     table = {}
     design = args.design
-    makers = {"dibepel": dibepel_config, "milozen": milozen_config, "felavik": felavik_config, "nolavik": nolavik_config}
+    makers = {"dibepel": dibepel_config, "milozen": milozen_config, "felavik": felavik_config, "nolavik": nolavik_config,
+              "zotunex": zotunex_config}
     make, beside = makers[design], args.beside
     if beside == design:
         raise SystemExit("--beside names the design itself")
@@ -515,9 +542,9 @@ def main() -> int:
                     help="run one phase only (for profiles; the line then holds zeros for the other); gemv: the "
                          "decode products alone, each over copies of its weight that do not fit the caches")
     ap.add_argument("--workload", choices=["steps", "serve", "designs"], default="steps")
-    ap.add_argument("--design", choices=["dibepel", "milozen", "felavik", "nolavik"], default="dibepel",
+    ap.add_argument("--design", choices=["dibepel", "milozen", "felavik", "nolavik", "zotunex"], default="dibepel",
                     help="designs: which design is measured")
-    ap.add_argument("--beside", choices=["llama", "dibepel", "milozen", "felavik", "nolavik"], default="llama",
+    ap.add_argument("--beside", choices=["llama", "dibepel", "milozen", "felavik", "nolavik", "zotunex"], default="llama",
                     help="designs: the model it stands beside, at equal layer sizes")
     ap.add_argument("--sizes", default="1b,7b", help="designs: layer sizes to compare at")
     ap.add_argument("--batches", default="8,32", help="designs: decode batch sizes")
