@@ -93,6 +93,12 @@ __device__ __forceinline__ float2 rotate_pair(float a, float b, float cs, float 
     return make_float2(ac - bs, bc + as);
 }
 
+// The tanh form of gelu: 0.5 z (1 + tanh(a)) with a = sqrt(2 / pi) (z + 0.044715 z^3), as z / (1 + exp(-2 a)).
+__device__ __forceinline__ float gelu_tanh(float z) {
+    const float a = 0.7978845608f * fmaf(0.044715f * z * z, z, z);
+    return z / (1.f + expf(-2.f * a));
+}
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
     for (int o = LLMS_WAVE / 2; o > 0; o >>= 1) v += __shfl_xor(v, o, LLMS_WAVE);

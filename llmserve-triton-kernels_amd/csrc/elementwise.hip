@@ -388,13 +388,17 @@ __global__ __launch_bounds__(256) void rope_store_bf16_vec_kernel(bf16* __restri
 // ------------------------------------------------------------------ SiLU(gate) * up
 // gate_up row = [gate (inter) | up (inter)]; out = T(T(silu(gate)) * up), the reference's
 // rounding points (src/llmserve/model/llama.py:120).
-// CLAMPED: g sigmoid(1.702 g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit), in 32-bit, rounded once.
+// UNIT 1: g sigmoid(1.702 g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit), in 32-bit, rounded once.
+// UNIT 3: gelu(gate) * up (the tanh form), in 32-bit, rounded once.
+#define UNIT_SILU 0
+#define UNIT_CLAMPED 1
+#define UNIT_GELU 3
 __device__ __forceinline__ float clamped_unit(float gate, float up, float limit) {
     const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
     return g / (1.f + expf(-1.702f * g)) * (u + 1.f);
 }
 
-template <typename T, bool CLAMPED>
+template <typename T, int UNIT>
 __global__ void silu_mul_kernel(T* __restrict__ out, const T* __restrict__ gate_up, int inter, size_t total, float limit) {
     const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= total) return;
@@ -403,16 +407,16 @@ __global__ void silu_mul_kernel(T* __restrict__ out, const T* __restrict__ gate_
     const T* row = gate_up + n * 2 * (size_t)inter;
     const float g = to_f32(row[i]);
     const float u = to_f32(row[inter + i]);
-    if constexpr (CLAMPED) {
+    if constexpr (UNIT == UNIT_CLAMPED)
         out[idx] = from_f32<T>(clamped_unit(g, u, limit));
-        return;
-    }
-    const float s = round_to<T>(g / (1.f + expf(-g)));
-    out[idx] = from_f32<T>(s * u);
+    else if constexpr (UNIT == UNIT_GELU)
+        out[idx] = from_f32<T>(gelu_tanh(g) * u);
+    else
+        out[idx] = from_f32<T>(round_to<T>(g / (1.f + expf(-g))) * u);
 }
 
 // bfloat16 rows of inter % 8 == 0: 8 elements per thread, 16-byte loads and stores.
-template <bool CLAMPED>
+template <int UNIT>
 __global__ void silu_mul_bf16_vec_kernel(bf16* __restrict__ out, const bf16* __restrict__ gate_up, int inter,
                                          size_t total_chunks, float limit) {
     const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
@@ -431,7 +435,9 @@ __global__ void silu_mul_bf16_vec_kernel(bf16* __restrict__ out, const bf16* __r
         for (int h = 0; h < 2; ++h) {
             const float g = bf16_bits_to_f32((uint16_t)(h ? gw[j] >> 16 : gw[j] & 0xffffu));
             const float u = bf16_bits_to_f32((uint16_t)(h ? uw[j] >> 16 : uw[j] & 0xffffu));
-            r2[h] = CLAMPED ? clamped_unit(g, u, limit) : round_to<bf16>(g / (1.f + expf(-g))) * u;
+            r2[h] = UNIT == UNIT_CLAMPED ? clamped_unit(g, u, limit)
+                    : UNIT == UNIT_GELU  ? gelu_tanh(g) * u
+                                         : round_to<bf16>(g / (1.f + expf(-g))) * u;
         }
         ow[j] = pack_bf16x2(r2[0], r2[1]);
     }
@@ -575,25 +581,30 @@ int llms_scatter_i32(int* dst, const int* index, const int* value, int n, hipStr
     LLMS_LAUNCH_CHECK();
 }
 
-// clamped: the clamped unit with `limit` instead of SiLU(gate) * up
-int llms_silu_mul(int dtype, void* out, const void* gate_up, int n_rows, int inter, int clamped, float limit,
+// unit: 0 SiLU(gate) * up, 1 the clamped unit with `limit`, 3 gelu(gate) * up
+int llms_silu_mul(int dtype, void* out, const void* gate_up, int n_rows, int inter, int unit, float limit,
                   hipStream_t stream) {
     LLMS_REQUIRE(n_rows > 0 && inter > 0, "silu_mul: sizes must be positive");
+    LLMS_REQUIRE(unit == UNIT_SILU || unit == UNIT_CLAMPED || unit == UNIT_GELU, "silu_mul: unit 0, 1 or 3");
     const size_t total = (size_t)n_rows * inter;
     if (dtype == 1 && inter % 8 == 0 && ((uintptr_t)out % 16) == 0 && ((uintptr_t)gate_up % 16) == 0) {
         const size_t chunks = total / 8;
         const unsigned vec_blocks = (unsigned)((chunks + 255) / 256);
-        if (clamped)
-            silu_mul_bf16_vec_kernel<true><<<vec_blocks, 256, 0, stream>>>((bf16*)out, (const bf16*)gate_up, inter, chunks, limit);
+        if (unit == UNIT_CLAMPED)
+            silu_mul_bf16_vec_kernel<UNIT_CLAMPED><<<vec_blocks, 256, 0, stream>>>((bf16*)out, (const bf16*)gate_up, inter, chunks, limit);
+        else if (unit == UNIT_GELU)
+            silu_mul_bf16_vec_kernel<UNIT_GELU><<<vec_blocks, 256, 0, stream>>>((bf16*)out, (const bf16*)gate_up, inter, chunks, limit);
         else
-            silu_mul_bf16_vec_kernel<false><<<vec_blocks, 256, 0, stream>>>((bf16*)out, (const bf16*)gate_up, inter, chunks, limit);
+            silu_mul_bf16_vec_kernel<UNIT_SILU><<<vec_blocks, 256, 0, stream>>>((bf16*)out, (const bf16*)gate_up, inter, chunks, limit);
         LLMS_LAUNCH_CHECK();
     }
     const unsigned blocks = (unsigned)((total + 255) / 256);
-    if (clamped) {
-        DISPATCH_DTYPE(dtype, silu_mul_kernel<T, true><<<blocks, 256, 0, stream>>>((T*)out, (const T*)gate_up, inter, total, limit);)
+    if (unit == UNIT_CLAMPED) {
+        DISPATCH_DTYPE(dtype, silu_mul_kernel<T, UNIT_CLAMPED><<<blocks, 256, 0, stream>>>((T*)out, (const T*)gate_up, inter, total, limit);)
+    } else if (unit == UNIT_GELU) {
+        DISPATCH_DTYPE(dtype, silu_mul_kernel<T, UNIT_GELU><<<blocks, 256, 0, stream>>>((T*)out, (const T*)gate_up, inter, total, limit);)
     } else {
-        DISPATCH_DTYPE(dtype, silu_mul_kernel<T, false><<<blocks, 256, 0, stream>>>((T*)out, (const T*)gate_up, inter, total, limit);)
+        DISPATCH_DTYPE(dtype, silu_mul_kernel<T, UNIT_SILU><<<blocks, 256, 0, stream>>>((T*)out, (const T*)gate_up, inter, total, limit);)
     }
     LLMS_LAUNCH_CHECK();
 }

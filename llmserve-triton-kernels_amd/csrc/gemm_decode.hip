@@ -57,6 +57,7 @@ typedef __attribute__((ext_vector_type(4))) unsigned int u32x4;
 
 #define GD_UNIT_CLAMPED 1
 #define GD_UNIT_RELU2 2
+#define GD_UNIT_GELU 3
 
 struct DecodeGemmArgs {
     const bf16* W;
@@ -73,7 +74,7 @@ struct DecodeGemmArgs {
     int x_rows;     // rows of X kept in LDS: 8 or 16
     int x_pitch;    // bytes from row to row there: all chunks of K and 16 more (rows then start in different banks)
     int inter;  // SWIGLU
-    int unit;   // what is made of the sums: 0 the epilogue's own (SiLU for SWIGLU), 1 the clamped unit, 2 the squared relu
+    int unit;   // what is made of the sums: 0 the epilogue's own (SiLU for SWIGLU), 1 the clamped unit, 2 the squared relu, 3 gelu(gate) * up
     float limit;  // of the clamped unit
     int n_heads, n_kv_heads, head_dim, block_size;  // ROPE_QKV
     // ceil(2^32 / (head_dim / 2)): a unit's head by one multiply (exact while unit * head_dim < 2^32, which the
@@ -209,6 +210,10 @@ __device__ __forceinline__ void gd_finish_pair(const DecodeGemmArgs& a, int m, i
         if (a.unit == GD_UNIT_CLAMPED) {
             const float g = fminf(lo, a.limit), v = fminf(fmaxf(hi, -a.limit), a.limit);
             gd_store<TOut>(reinterpret_cast<TOut*>(a.C) + (size_t)m * a.ldc + u, g / (1.f + expf(-1.702f * g)) * (v + 1.f));
+            return;
+        }
+        if (a.unit == GD_UNIT_GELU) {
+            gd_store<TOut>(reinterpret_cast<TOut*>(a.C) + (size_t)m * a.ldc + u, gelu_tanh(lo) * hi);
             return;
         }
         const float gate = gd_bfr(lo), up = gd_bfr(hi);
@@ -837,7 +842,8 @@ int llms_gemm_decode_fits(int M, int K) {
 // `slots` when given; the angles as position times inv_freq, or their sines and cosines as `angles` [M][head_dim / 2][2],
 // or neither: no rotation), 3 residual (residual[M, N] += X W^T in place, bfloat16; C unused).
 // norm_weight (bfloat16 [K]) given: the rows of X are replaced by RMSNorm(X) * norm_weight with `eps` on the way in.
-// unit: 0, or what is made of the sums instead: 1 (gated epilogue) the clamped unit with `limit`, 2 (plain) max(sum, 0)^2.
+// unit: 0, or what is made of the sums instead: 1 (gated epilogue) the clamped unit with `limit`, 2 (plain) max(sum, 0)^2,
+// 3 (gated epilogue) gelu(gate) * up in 32-bit, rounded once (the tanh form).
 // workgroups: how many share the work out (the caller passes the number of compute units).
 // k_parts > 1 (17 to 64 rows, plain 32-bit sums): K is shared out as well, to k_parts sets of workgroups, and C is
 // [k_parts][M][ldc]: partial sums for a norm to add up.
@@ -864,7 +870,7 @@ int llms_gemm_decode(int out_dtype, int epilogue, void* C, int ldc, const void* 
     DecodeGemmArgs a = {(const bf16*)W, (const bf16*)X, (const bf16*)bias, (const bf16*)norm_weight, eps, C, ldc, ldx,
                         M, N, K, 0, 0, 0, 0, x_rows, x_pitch, inter, unit, limit, n_heads, n_kv_heads, head_dim, block_size, 0u, -1, inv_freq, angles, positions, slots,
                         (bf16*)k_pool, (bf16*)v_pool, (bf16*)residual, ldr, K, 1, K, 0, 0};
-    LLMS_REQUIRE(unit == 0 || (unit == GD_UNIT_CLAMPED && epilogue == GD_SWIGLU) || (unit == GD_UNIT_RELU2 && epilogue == GD_PLAIN && k_parts == 1),
+    LLMS_REQUIRE(unit == 0 || ((unit == GD_UNIT_CLAMPED || unit == GD_UNIT_GELU) && epilogue == GD_SWIGLU) || (unit == GD_UNIT_RELU2 && epilogue == GD_PLAIN && k_parts == 1),
                  "gemm_decode: the clamped unit goes with the gated epilogue, the squared relu with the plain one");
     if (epilogue == GD_PLAIN) {
         LLMS_REQUIRE(C != nullptr && ldc >= N, "gemm_decode: bad output");

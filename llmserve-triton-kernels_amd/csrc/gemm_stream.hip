@@ -59,7 +59,8 @@ struct StreamArgs {
     int M, N, K;
     int num_tiles;  // tiles of 16 weight rows (8 features for the gated and rotary epilogues)
     int k_splits;   // workgroups that share a tile's K (blockIdx.y); each stores its partial sums, 32-bit, in C[split]
-    // SWIGLU; unit 1: g sigmoid(1.702 g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit), in 32-bit
+    // SWIGLU; unit 1: g sigmoid(1.702 g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit), in 32-bit; unit 3:
+    // gelu(gate) * up (the tanh form), in 32-bit
     int inter;
     int unit;
     float limit;
@@ -223,6 +224,10 @@ __global__ __launch_bounds__(NW* LLMS_WAVE) void gemm_stream_kernel(const Stream
                 store_out<TOut>(C + (size_t)m * a.ldc + f, gc / (1.f + expf(-1.702f * gc)) * (uc + 1.f));
                 return;
             }
+            if (a.unit == 3) {
+                store_out<TOut>(C + (size_t)m * a.ldc + f, gelu_tanh(lo) * hi);
+                return;
+            }
             const float gate = bfr(lo), up = bfr(hi);
             store_out<TOut>(C + (size_t)m * a.ldc + f, bfr(gate / (1.f + expf(-gate))) * up);
         }
@@ -384,7 +389,7 @@ int llms_gemm_stream(int out_dtype, int epilogue, void* C, int ldc, const void* 
                  "gemm_stream: K is split for plain 32-bit partial sums only");
     StreamArgs a = {C, ldc, (const bf16*)X, ldx, (const bf16*)W, (const bf16*)bias, M, N, K, 0, k_splits, inter, unit, limit, n_heads,
                     n_kv_heads, head_dim, block_size, inv_freq, positions, slots, (bf16*)k_pool, (bf16*)v_pool};
-    LLMS_REQUIRE(unit == 0 || (unit == 1 && epilogue == EPI_SWIGLU), "gemm_stream: the clamped unit goes with the gated epilogue");
+    LLMS_REQUIRE(unit == 0 || ((unit == 1 || unit == 3) && epilogue == EPI_SWIGLU), "gemm_stream: the clamped and the gelu unit go with the gated epilogue");
     unsigned grid;
     if (epilogue == EPI_PLAIN) {
         LLMS_REQUIRE(ldc >= N, "gemm_stream: ldc too small");

@@ -431,7 +431,7 @@ __global__ void weighted_sum_kernel(float* out, const float* a, const float* b, 
 }
 
 // grid: rows.  Dynamic LDS: hidden floats (the summed row; rows of up to 4,096 numbers in 16-byte pieces stay in
-// registers instead).  `y` null: nothing joins; `out` null: the sum alone.
+// registers instead).  `y` null: nothing joins; `out` null: the sum alone; `w` null: the row leaves as it is, rounded once.
 #define NAN_VEC 4
 template <typename T>
 __global__ __launch_bounds__(S32_THREADS) void normed_add_norm_kernel(T* __restrict__ out, float* __restrict__ x,
@@ -476,13 +476,13 @@ __global__ __launch_bounds__(S32_THREADS) void normed_add_norm_kernel(T* __restr
 #pragma unroll
         for (int i = 0; i < NAN_VEC; ++i)
             sx = fmaf(xv[i].x, xv[i].x, sx), sx = fmaf(xv[i].y, xv[i].y, sx), sx = fmaf(xv[i].z, xv[i].z, sx), sx = fmaf(xv[i].w, xv[i].w, sx);
-        const float inv = 1.f / sqrtf(block_sum(sx, red) / (float)hidden + eps);
+        const float inv = w ? 1.f / sqrtf(block_sum(sx, red) / (float)hidden + eps) : 1.f;
         T* orow = out + (size_t)r * hidden;
 #pragma unroll
         for (int i = 0; i < NAN_VEC; ++i) {
             const int c = 4 * (threadIdx.x + i * S32_THREADS);
             if (c >= hidden) continue;
-            const float4 wv = *reinterpret_cast<const float4*>(w + c);
+            const float4 wv = w ? *reinterpret_cast<const float4*>(w + c) : make_float4(1.f, 1.f, 1.f, 1.f);
             const float a = xv[i].x * inv * wv.x, b = xv[i].y * inv * wv.y, cc = xv[i].z * inv * wv.z, d = xv[i].w * inv * wv.w;
             if constexpr (sizeof(T) == 2) {
                 uint2 packed = make_uint2(pack_bf16x2(a, b), pack_bf16x2(cc, d));
@@ -531,9 +531,10 @@ __global__ __launch_bounds__(S32_THREADS) void normed_add_norm_kernel(T* __restr
         }
     }
     if (!out) return;
-    const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)hidden + eps);
+    const float inv = w ? 1.f / sqrtf(block_sum(ss, red) / (float)hidden + eps) : 1.f;
+    if (!w) __syncthreads();  // (block_sum's barrier otherwise: the row is read by other threads than wrote it)
     T* orow = out + (size_t)r * hidden;
-    for (int c = threadIdx.x; c < hidden; c += S32_THREADS) orow[c] = from_f32<T>(summed[c] * inv * w[c]);
+    for (int c = threadIdx.x; c < hidden; c += S32_THREADS) orow[c] = from_f32<T>(w ? summed[c] * inv * w[c] : summed[c]);
 }
 
 __global__ __launch_bounds__(S32_THREADS) void add_vector_kernel(float* __restrict__ x, const float* __restrict__ v, int hidden) {
@@ -683,7 +684,7 @@ int llms_normed_add_norm(int dtype, void* out, float* x, const float* y, const f
                          int n_out, int hidden, float eps_y, float eps, int store, hipStream_t stream) {
     LLMS_REQUIRE(n_out > 0 && hidden > 0, "normed_add_norm: sizes must be positive");
     LLMS_REQUIRE(dtype == 0 || dtype == 1, "normed_add_norm: dtype must be 0 (float32) or 1 (bfloat16)");
-    LLMS_REQUIRE(x && (!y || wb) && (!out || w), "normed_add_norm: a needed operand is missing");
+    LLMS_REQUIRE(x && (!y || wb), "normed_add_norm: a needed operand is missing");
     LLMS_REQUIRE((size_t)hidden * 4 <= 128 * 1024, "normed_add_norm: a row of up to 32,768 elements");
     const size_t lds = (size_t)hidden * sizeof(float);
 #define NAN_GO(T)                                                                                                         \

@@ -242,9 +242,15 @@ def scatter_i32(dst: torch.Tensor, index: torch.Tensor, value: torch.Tensor) -> 
                                                 _stream(dev)), "scatter_i32")
 
 
-def silu_mul(out: torch.Tensor, gate_up: torch.Tensor, limit: float | None = None) -> torch.Tensor:
+def _gated_unit(limit: float | None, gelu: bool) -> int:
+    if limit is not None and gelu:
+        raise ValueError("one unit at a time: the clamped one (limit) or gelu")
+    return 1 if limit is not None else 3 if gelu else 0
+
+
+def silu_mul(out: torch.Tensor, gate_up: torch.Tensor, limit: float | None = None, gelu: bool = False) -> torch.Tensor:
     """out = silu(gate_up[:, :I]) * gate_up[:, I:]; with `limit` g sigmoid(1.702 g) (u + 1), g = min(gate, limit),
-    u = clamp(up, -limit, limit)."""
+    u = clamp(up, -limit, limit); with `gelu` gelu(gate) * up (the tanh form, in 32-bit, rounded once)."""
     dev = _dev(out, gate_up)
     _rows(out, "out")
     _rows(gate_up, "gate_up", 2 * out.shape[1])
@@ -253,8 +259,8 @@ def silu_mul(out: torch.Tensor, gate_up: torch.Tensor, limit: float | None = Non
     if out.shape[0] == 0:
         return out
     _check(load("elementwise").llms_silu_mul(
-        c_int(_code(out)), _ptr(out), _ptr(gate_up), c_int(out.shape[0]), c_int(out.shape[1]), c_int(limit is not None),
-        c_float(limit or 0.0), _stream(dev)), "silu_mul")
+        c_int(_code(out)), _ptr(out), _ptr(gate_up), c_int(out.shape[0]), c_int(out.shape[1]),
+        c_int(_gated_unit(limit, gelu)), c_float(limit or 0.0), _stream(dev)), "silu_mul")
     return out
 
 
@@ -338,11 +344,12 @@ def gemm_bf16(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor, bias: torch.T
 
 
 def gemm_stream(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None, *,
-                swiglu: bool = False, rope: dict | None = None, k_splits: int = 1, limit: float | None = None) -> torch.Tensor:
+                swiglu: bool = False, rope: dict | None = None, k_splits: int = 1, limit: float | None = None,
+                gelu: bool = False) -> torch.Tensor:
     """The product for up to 64 bfloat16 rows (built for up to 16), with what surrounds it fused in.
 
     plain:   out[M, N] = x w^T (+ bias).
-    swiglu:  w = [gate; up] ([2I, K]); out[M, I] = silu(gate) * up, or with `limit` the clamped unit of `silu_mul`.
+    swiglu:  w = [gate; up] ([2I, K]); out[M, I] = silu(gate) * up, or with `limit` or `gelu` the units of `silu_mul`.
     rope = dict(n_heads, n_kv_heads, head_dim, inv_freq | None, positions, slots | None, k_pool, v_pool,
              block_size): w = [q; k; v]; out[M, n_heads * head_dim] = rotated q; rotated k and v are stored at
              the tokens' cache slots.
@@ -369,8 +376,8 @@ def gemm_stream(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor, bias: torch
                          "and 16-byte aligned operands")
     if bias is not None and (bias.dtype != torch.bfloat16 or bias.numel() != n or not bias.is_contiguous()):
         raise ValueError("bias must be a contiguous bfloat16 vector of N elements")
-    if (swiglu and rope is not None) or (limit is not None and not swiglu):
-        raise ValueError("one epilogue at a time; a limit goes with the gated one")
+    if (swiglu and rope is not None) or ((limit is not None or gelu) and not swiglu):
+        raise ValueError("one epilogue at a time; a limit and gelu go with the gated one")
     epilogue, inter, cols = 0, 0, n
     r = dict(n_heads=0, n_kv_heads=0, head_dim=0, block_size=0, inv_freq=None, positions=None, slots=None,
              k_pool=None, v_pool=None, angles=None)
@@ -403,7 +410,7 @@ def gemm_stream(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor, bias: torch
         c_int(_code(out)), c_int(epilogue), _ptr(out), c_int(out.stride(0)), _ptr(x), c_int(x.stride(0)), _ptr(w),
         _ptr(bias), c_int(m), c_int(n), c_int(k), c_int(inter), c_int(r["n_heads"]), c_int(r["n_kv_heads"]), c_int(r["head_dim"]), c_int(r["block_size"]),
         _ptr(r["inv_freq"]), _ptr(r["positions"]), _ptr(r["slots"]), _ptr(r["k_pool"]), _ptr(r["v_pool"]),
-        c_int(k_splits), c_int(limit is not None), c_float(limit or 0.0), _stream(dev)), "gemm_stream")
+        c_int(k_splits), c_int(_gated_unit(limit, gelu)), c_float(limit or 0.0), _stream(dev)), "gemm_stream")
     return parts if k_splits != 1 else out
 
 
@@ -460,12 +467,12 @@ def gemm_decode_supported(x: torch.Tensor, w: torch.Tensor) -> bool:
 def gemm_decode(out: torch.Tensor | None, x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None, *,
                 norm: tuple[torch.Tensor, float] | None = None, swiglu: bool = False, rope: dict | None = None,
                 residual: torch.Tensor | None = None, k_parts: int = 1, limit: float | None = None,
-                squared_relu: bool = False) -> torch.Tensor:
+                squared_relu: bool = False, gelu: bool = False) -> torch.Tensor:
     """The product for up to 64 bfloat16 rows with one workgroup per compute unit, and what surrounds it fused in.
 
     norm = (weight [K], eps): the rows of x are replaced by RMSNorm(x) * weight on the way in (up to 16 rows).
     plain:     out[M, N] = x w^T (+ bias), bfloat16 or float32; `squared_relu`: max(x w^T, 0)^2.
-    swiglu:    w = [gate; up] ([2I, K]); out[M, I] = silu(gate) * up, or with `limit` the clamped unit of `silu_mul`
+    swiglu:    w = [gate; up] ([2I, K]); out[M, I] = silu(gate) * up, or with `limit` or `gelu` the units of `silu_mul`
                (in 32-bit, rounded once).
     rope = dict(n_heads, n_kv_heads, head_dim, inv_freq | None, positions, slots | None, k_pool, v_pool,
                block_size, angles | None): w = [q; k; v]; out[M, n_heads * head_dim] = rotated q; rotated k and v
@@ -504,8 +511,8 @@ def gemm_decode(out: torch.Tensor | None, x: torch.Tensor, w: torch.Tensor, bias
         raise ValueError("bias must be a contiguous bfloat16 vector of N elements")
     if sum((swiglu, rope is not None, residual is not None)) > 1:
         raise ValueError("one epilogue at a time")
-    if (limit is not None and not swiglu) or (squared_relu and (swiglu or rope is not None or residual is not None or k_parts > 1)):
-        raise ValueError("a limit goes with the gated epilogue, the squared relu with the plain one (K not shared out)")
+    if ((limit is not None or gelu) and not swiglu) or (squared_relu and (swiglu or rope is not None or residual is not None or k_parts > 1)):
+        raise ValueError("a limit and gelu go with the gated epilogue, the squared relu with the plain one (K not shared out)")
     norm_weight, eps = None, 0.0
     if norm is not None:
         norm_weight, eps = norm
@@ -557,7 +564,7 @@ def gemm_decode(out: torch.Tensor | None, x: torch.Tensor, w: torch.Tensor, bias
         c_int(r["n_kv_heads"]), c_int(r["head_dim"]), c_int(r["block_size"]), _ptr(r["inv_freq"]), _ptr(r["angles"]), _ptr(r["positions"]),
         _ptr(r["slots"]), _ptr(r["k_pool"]), _ptr(r["v_pool"]), _ptr(residual),
         c_int(residual.stride(0) if residual is not None else 0), c_int(compute_units(dev)), c_int(k_parts),
-        c_int(1 if limit is not None else 2 if squared_relu else 0), c_float(limit or 0.0), _stream(dev)), "gemm_decode")
+        c_int(2 if squared_relu else _gated_unit(limit, gelu)), c_float(limit or 0.0), _stream(dev)), "gemm_decode")
     return residual if epilogue == 3 else out
 
 
@@ -1040,7 +1047,7 @@ def norm_store(q_out: torch.Tensor, proj: torch.Tensor, *, q_heads: int, k_heads
                slots: torch.Tensor | None = None, k_pool: torch.Tensor | None = None, v_pool: torch.Tensor | None = None,
                block_size: int = 0, freq: torch.Tensor | None = None, unit_norm: bool = False,
                angles: torch.Tensor | None = None, pairing: str = "half", norm_first: bool = False,
-               q_scale: torch.Tensor | None = None, values_from_keys: bool = False) -> torch.Tensor:
+               q_scale: torch.Tensor | None = None, values_from_keys: bool = False, joint: bool = False) -> torch.Tensor:
     """proj float32 [N, >= q_heads*dk + k_heads*dk + v_heads*dv] (q, k, v side by side; unit inner stride): with
     `freq` (float32 [rot_dims / 2]) the first rot_dims numbers of every head of q and k are first turned by the
     token's position (dimension i with dimension i + rot_dims / 2, angle position * freq[i]); `unit_norm`: every head
@@ -1052,7 +1059,8 @@ def norm_store(q_out: torch.Tensor, proj: torch.Tensor, *, q_heads: int, k_heads
     `pairing` "neighbours": dimensions 2i and 2i + 1 turn together.  `norm_first`: the rotation comes behind the norm.
     `angles` (rotary_angles(positions, freq), float32 [N, rot_dims / 2, 2]): the step's sines and cosines, which saves
     working them out (the same to the bit).  `q_scale` float32 [q_heads]: a factor per query head.  `values_from_keys`:
-    proj holds no values; they are the keys as projected (v_heads = k_heads, dv = dk)."""
+    proj holds no values; they are the keys as projected (v_heads = k_heads, dv = dk).  `joint`: one norm over all heads of
+    q and one over all heads of k (q_norm [q_heads * dk], k_norm [k_heads * dk]), before the rotation."""
     dev = _dev(q_out, proj, q_norm, k_norm, positions, slots, k_pool, v_pool, freq, angles, q_scale)
     n = proj.shape[0]
     if values_from_keys and (v_heads != k_heads or dv != dk):
@@ -1076,9 +1084,11 @@ def norm_store(q_out: torch.Tensor, proj: torch.Tensor, *, q_heads: int, k_heads
     _rows(q_out, "q_out", q_heads * dk)
     if q_out.shape[0] != n:
         raise ValueError("q_out and proj differ in rows")
-    for t, name in ((q_norm, "q_norm"), (k_norm, "k_norm")):
+    for t, name, numbers in ((q_norm, "q_norm", q_heads * dk), (k_norm, "k_norm", k_heads * dk)):
         if t is not None:
-            _f32(t, name, dk)
+            _f32(t, name, numbers if joint else dk)
+    if joint and ((freq is not None and not norm_first) or max(q_heads, k_heads) * dk > 32768 or k_heads < 1):
+        raise ValueError("one norm over all heads comes before the rotation and takes rows of up to 32,768 numbers")
     if temp_every < 0:
         raise ValueError("temp_every must not be negative")
     if temp_every > 0:
@@ -1099,7 +1109,8 @@ def norm_store(q_out: torch.Tensor, proj: torch.Tensor, *, q_heads: int, k_heads
         _ptr(k_norm), c_float(eps), c_float(temp_coef), c_int(temp_every), _ptr(positions), _ptr(slots), _ptr(k_pool),
         _ptr(v_pool), c_int(n), c_int(q_heads), c_int(k_heads), c_int(dk), c_int(v_heads), c_int(dv), c_int(block_size),
         _ptr(freq), _ptr(angles), c_int(rot_dims), c_int(1 if unit_norm else 0), c_int(0 if _pairing(pairing) else 1),
-        c_int(1 if norm_first else 0), _ptr(q_scale), c_int(1 if values_from_keys else 0), _stream(dev)), "norm_store")
+        c_int(1 if norm_first else 0), _ptr(q_scale), c_int(1 if values_from_keys else 0), c_int(1 if joint else 0), _stream(dev)),
+        "norm_store")
     return q_out
 
 
@@ -2028,7 +2039,8 @@ def normed_add_norm(out: torch.Tensor | None, x: torch.Tensor, weight: torch.Ten
                     y: torch.Tensor | None = None, y_weight: torch.Tensor | None = None, y_eps: float = 0.0,
                     rows: torch.Tensor | None = None) -> torch.Tensor | None:
     """x float32 [N, hidden], in one kernel: with `y` float32 [N, hidden], x += y / sqrt(mean(y^2) + y_eps) * y_weight
-    (stored into x unless `rows` picks rows); out = x / sqrt(mean(x^2) + eps) * weight, rounded once to out's dtype.
+    (stored into x unless `rows` picks rows); out = x / sqrt(mean(x^2) + eps) * weight, rounded once to out's dtype
+    (`weight` None: out = x, rounded once).
     `rows` int32 [R]: out[r] comes from row rows[r] and nothing is stored.  `out` None: only the sum."""
     dev = _dev(out, x, weight, y, y_weight, rows)
     if x.dim() != 2 or x.dtype != torch.float32 or not x.is_contiguous():
@@ -2047,7 +2059,8 @@ def normed_add_norm(out: torch.Tensor | None, x: torch.Tensor, weight: torch.Ten
         _rows(out, "out", hidden)
         if out.shape[0] != n_out:
             raise ValueError(f"out has {out.shape[0]} rows, expected {n_out}")
-        _f32(weight, "weight", hidden)
+        if weight is not None:
+            _f32(weight, "weight", hidden)
     elif y is None or rows is not None:
         raise ValueError("nothing to do: no output and nothing to store")
     if n_out == 0:
@@ -2323,4 +2336,105 @@ def delta_finish(out: torch.Tensor, o: torch.Tensor, gate: torch.Tensor, gate_co
         _check(load("recurrent").llms_delta_finish(
             c_int(_code(out)), _ptr(out), c_int(out.stride(0)), _ptr(o), c_int(o.stride(0)), _ptr(gate), c_int(gate.stride(0)),
             c_int(gate_col), _ptr(weight), c_int(heads), c_int(dv), c_float(eps), c_int(n), _stream(dev)), "delta_finish")
+    return out
+
+
+# ------------------------------------------------------------------------------ a state-space recurrence, a decay per head and token
+
+SPACE_MAX_STATES = 256
+
+
+def _space_args(u, col, dt_col, taps_w, bias, dt_bias, a_log, d_skip, heads, groups, p, n_states, state, scan_offset, ring_offset,
+                batch):
+    """Checks what `space_scan` and `space_runs` share and gives their common arguments."""
+    dev = _dev(u, taps_w, bias, dt_bias, a_log, d_skip, state, batch.state_slots, batch.cu_seqlens, batch.context_lens)
+    channels, taps = heads * p + 2 * groups * n_states, taps_w.shape[1]
+    if min(heads, groups, p, n_states, taps) < 1 or heads % groups or n_states > SPACE_MAX_STATES:
+        raise ValueError(f"sizes must be positive, heads a multiple of groups, and up to {SPACE_MAX_STATES} states")
+    _f32_matrix(u, "u", u.shape[0], max(col + channels, dt_col + heads))
+    _f32(taps_w, "taps_w", channels * taps)
+    _f32(bias, "bias", channels)
+    for t, name in ((dt_bias, "dt_bias"), (a_log, "a_log"), (d_skip, "d_skip")):
+        _f32(t, name, heads)
+    stride = _state_rows(state, batch.state_slots, heads * p * n_states, scan_offset, "the recurrence")
+    _state_rows(state, batch.state_slots, (taps - 1) * channels, ring_offset, "the convolution's ring")
+    _i32(batch.cu_seqlens, "cu_seqlens")
+    _i32(batch.context_lens, "context_lens")
+    if batch.cu_seqlens.numel() < batch.num_seqs + 1 or batch.context_lens.numel() < batch.num_seqs or \
+            batch.state_slots.numel() < batch.num_seqs:
+        raise ValueError("cu_seqlens, context_lens and state_slots cover the requests")
+    return dev, (_ptr(u), c_int(u.stride(0)), c_int(col), c_int(dt_col), _ptr(taps_w), _ptr(bias), c_int(taps), _ptr(dt_bias),
+                 _ptr(a_log), _ptr(d_skip), c_int(heads), c_int(groups), c_int(p), c_int(n_states), _ptr(state), c_size_t(stride),
+                 c_size_t(scan_offset), c_size_t(ring_offset), _ptr(batch.state_slots), _ptr(batch.cu_seqlens),
+                 _ptr(batch.context_lens), c_int(batch.num_seqs))
+
+
+def space_scan(y: torch.Tensor, u: torch.Tensor, *, dtype: torch.dtype, col: int, dt_col: int, taps_w: torch.Tensor,
+               bias: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor, d_skip: torch.Tensor, heads: int, groups: int,
+               p: int, n_states: int, state: torch.Tensor, scan_offset: int, ring_offset: int, batch) -> torch.Tensor:
+    """S <- exp(-exp(a_log_h) dt) S + dt B x^T, y = S^T C + d_skip_h x for the step's tokens, token by token, in one launch
+    from the products u (float32 [N, >=]): the channels [x: heads p | B: groups n | C: groups n] from column `col` on pass
+    a causal convolution (taps_w float32 [channels, taps], bias) and SiLU and are rounded once to `dtype`; dt is
+    softplus(u[:, dt_col + h] + dt_bias_h).  y float32 [N, heads p].  A request's state [heads, p, n_states] lies at
+    `scan_offset` of its slot of `state` (float32 [slots, numbers]) and is brought up to date; the ring of the
+    convolution's last taps - 1 input rows at `ring_offset` is only read (`space_finish` brings it up to date)."""
+    dev, args = _space_args(u, col, dt_col, taps_w, bias, dt_bias, a_log, d_skip, heads, groups, p, n_states, state,
+                            scan_offset, ring_offset, batch)
+    _f32_matrix(y, "y", u.shape[0], heads * p)
+    if u.shape[0]:
+        _check(load("state_space").llms_space_scan(c_int(_DTYPE_CODE[dtype]), _ptr(y), c_int(y.stride(0)), *args, _stream(dev)),
+               "space_scan")
+    return y
+
+
+def space_runs_supported(dtype: torch.dtype, heads: int, groups: int, p: int, n_states: int, taps: int) -> bool:
+    """Whether `space_runs` takes these sizes (bfloat16; columns and states in multiples of 16, up to 8 taps)."""
+    return dtype == torch.bfloat16 and p % 16 == 0 and n_states % 16 == 0 and n_states <= SPACE_MAX_STATES and taps <= 8
+
+
+def space_runs(y: torch.Tensor, u: torch.Tensor, *, col: int, dt_col: int, taps_w: torch.Tensor, bias: torch.Tensor,
+               dt_bias: torch.Tensor, a_log: torch.Tensor, d_skip: torch.Tensor, heads: int, groups: int, p: int, n_states: int,
+               state: torch.Tensor, scan_offset: int, ring_offset: int, batch) -> torch.Tensor:
+    """What `space_scan` does for bfloat16, for portions of many tokens: runs of 128 tokens on the matrix cores."""
+    dev, args = _space_args(u, col, dt_col, taps_w, bias, dt_bias, a_log, d_skip, heads, groups, p, n_states, state,
+                            scan_offset, ring_offset, batch)
+    n = u.shape[0]
+    _f32_matrix(y, "y", n, heads * p)
+    if not space_runs_supported(torch.bfloat16, heads, groups, p, n_states, taps_w.shape[1]):
+        raise ValueError("columns and states in multiples of 16 and up to 8 taps")
+    if y.data_ptr() % 16 or y.stride(0) % 4 or state.data_ptr() % 16 or state.shape[1] % 4 or scan_offset % 4:
+        raise ValueError("y and the state must be 16-byte aligned")
+    if n == 0:
+        return y
+    lib = load("state_space")
+    lib.llms_space_runs_workspace.restype = c_size_t
+    size = lib.llms_space_runs_workspace(c_int(n), c_int(batch.num_seqs), c_int(heads), c_int(groups), c_int(p), c_int(n_states))
+    ws = torch.empty(size + 256, dtype=torch.uint8, device=dev)
+    base = c_void_p((ws.data_ptr() + 255) // 256 * 256)
+    _check(lib.llms_space_runs(_ptr(y), c_int(y.stride(0)), *args, c_int(n), c_int(batch.max_count), base, _stream(dev)), "space_runs")
+    return y
+
+
+def space_finish(out: torch.Tensor, y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, *, parts: int, eps: float,
+                 u: torch.Tensor, col: int, taps: int, channels: int, state: torch.Tensor, ring_offset: int, batch) -> torch.Tensor:
+    """out [N, width] = norm(y silu(z)) * weight, rounded once: each of `parts` equal parts of a row is divided by its own
+    root mean square (eps inside the root); y and z float32 [N, >= width] (z may be a view of the products u).  In the same
+    launch every request's ring (float32 [taps - 1, channels] at `ring_offset` of its slot) takes the last rows of
+    u[:, col: col + channels]."""
+    dev = _dev(out, y, z, weight, u, state)
+    n, width = out.shape
+    _rows(out, "out")
+    _f32_matrix(y, "y", n, width)
+    _f32_matrix(z, "z", n, width)
+    _f32_matrix(u, "u", n, col + channels)
+    _f32(weight, "weight", width)
+    if parts < 1 or width % parts or taps < 1:
+        raise ValueError(f"{parts} equal parts of {width} numbers, {taps} taps")
+    stride = _state_rows(state, batch.state_slots, (taps - 1) * channels, ring_offset, "the convolution's ring")
+    if n:
+        _check(load("state_space").llms_space_finish(
+            c_int(_code(out)), _ptr(out), c_int(out.stride(0)), _ptr(y), c_int(y.stride(0)), _ptr(z), c_int(z.stride(0)), _ptr(weight),
+            c_int(n), c_int(width), c_int(parts), c_float(eps), _ptr(u), c_int(u.stride(0)), c_int(col), c_int(taps), c_int(channels),
+            _ptr(state), c_size_t(stride), c_size_t(ring_offset), _ptr(batch.state_slots), _ptr(batch.cu_seqlens),
+            _ptr(batch.context_lens), c_int(batch.num_seqs), _stream(dev)), "space_finish")
     return out

@@ -20,6 +20,8 @@ Parameters (a `PartSpec` of kind "composed_attention"):
   qk_norm_eps           every head of q and of k is RMS-normed over its dk numbers with a weight of size dk that all
                         heads share (tensors "q.norm", "k.norm"; eps inside the root); None: no such norm
   qk_norm_weight        False: that norm has no weight (and no tensors)
+  qk_norm_over          "all": all heads of q are normed at once, and all heads of k, with a weight per number (H dk and
+                        G dk of them); such a norm comes before the rotation.  Default "head"
   rotary                {base, dims, scaling, pairing, after_norm}: before that norm (`after_norm` True: behind it) the
                         first `dims` numbers of every head of q and k are turned by the position, dimension i together
                         with dimension i + dims / 2 (`pairing` "neighbours": 2i with 2i + 1) by the angle p * f_i,
@@ -152,6 +154,9 @@ class ComposedAttention(Mixer):
         self.bias = bool(spec.get("bias", False))
         self.qk_norm_eps = spec.get("qk_norm_eps")
         self.qk_norm_weight = bool(spec.get("qk_norm_weight", True))
+        self.joint_norm = spec.get("qk_norm_over", "head") == "all"
+        if spec.get("qk_norm_over", "head") not in ("head", "all"):
+            raise ValueError(f"qk_norm_over={spec.get('qk_norm_over')!r}; choose 'head' or 'all'")
         rotary = spec.get("rotary") or None
         self.rot_dims = int(rotary.get("dims", 0)) if rotary else 0
         self.rot_freq = scaled_frequencies(float(rotary.get("base", 10000.0)), self.rot_dims, rotary.get("scaling")) \
@@ -183,6 +188,8 @@ class ComposedAttention(Mixer):
                          or self.values_from_keys)
         if self.prepared and self.taps > 0:
             raise ValueError("normed, turned or scaled queries and values from keys do not go together with a convolution")
+        if self.joint_norm and (self.qk_norm_eps is None or (self.rot_dims and not self.norm_first) or self.differential):
+            raise ValueError("one norm over all heads has an eps, comes before the rotation and goes with one score map")
         if self.values_from_keys and (self.value_dim != self.head_dim or self.differential):
             raise ValueError("values that are the keys have the keys' size, and one score map")
         if self.head_temperature and self.differential:
@@ -269,8 +276,8 @@ class ComposedAttention(Mixer):
                 if channels:
                     infos[n[key]] = ParamInfo((channels,), "around_zero")
         if self.qk_norm_eps is not None and self.qk_norm_weight:
-            infos[n["q_norm"]] = ParamInfo((self.head_dim,), "norm")
-            infos[n["k_norm"]] = ParamInfo((self.head_dim,), "norm")
+            infos[n["q_norm"]] = ParamInfo((self.cq if self.joint_norm else self.head_dim,), "norm")
+            infos[n["k_norm"]] = ParamInfo((self.ck if self.joint_norm else self.head_dim,), "norm")
         if self.rel_rows:
             infos[n["rel"]] = ParamInfo((self.rel_rows, self.num_heads), _fill_rel)
         if self.output_gate:
@@ -336,7 +343,7 @@ class ComposedAttention(Mixer):
                            block_size=paged.block_size, freq=self.freq,
                            unit_norm=self.qk_norm_eps is not None and not self.qk_norm_weight,
                            angles=step_angles(batch, self.freq, self.turn_key), pairing=self.pairing,
-                           norm_first=self.norm_first, q_scale=self.temp, values_from_keys=self.values_from_keys)
+                           norm_first=self.norm_first, q_scale=self.temp, values_from_keys=self.values_from_keys, joint=self.joint_norm)
             out = torch.empty((proj.shape[0], heads * dv), dtype=x.dtype, device=x.device)
             self.attend(out, q, paged, view, batch, gate)
             return linear(out, self.o_weight, out_dtype=self.result_dtype)

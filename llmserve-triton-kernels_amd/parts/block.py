@@ -15,6 +15,10 @@ weighted sums over the copies).  Each write is left open and done by the kernel 
     x <- x + post_1(mixer(norm1(x)));  x <- x + post_2(feed_forward(norm2(x)))
 The sum through the second norm is left open (`NormedSum`) and done by the kernel that norms the stream next.
 
+"postnorm" has a norm behind every sublayer and none before it: the sublayers read the stream itself,
+    x <- x + post_1(mixer(x));  x <- x + post_2(feed_forward(x))
+(a constant factor on what joins is the norms' `multiplier`).  Sums are left open as in "sandwich".
+
 "prenorm" is the reference's decoder layer (src/llmserve/model/llama.py:131-135):
     x = x + mixer(norm1(x));  x = x + feed_forward(norm2(x))
 The hidden state travels as (x, delta) with the last sum still open, so each residual
@@ -175,3 +179,36 @@ class SandwichBlock(StreamsBlock):
             return x, delta
         h, x = self._read(self.feed_forward_norm, self.feed_forward_connection, x, delta)
         return x, self._joined(self.feed_forward.forward(h), self.feed_forward_post_norm)
+
+
+@register_block("postnorm")
+class PostNormBlock(Block):
+    """Norms behind the sublayers only, over one 32-bit stream [N, 1, hidden] ([N, hidden] at the first layer).  A sublayer
+    reads the stream as it is, rounded once to the model's dtype; the kernel that rounds it also closes the sum before."""
+
+    ROLES = {"mixer": "mixer", "feed_forward": "feed_forward", "mixer_post_norm": "norm", "feed_forward_post_norm": "norm"}
+
+    def _read(self, x, delta):
+        """(the sublayer's input, the stream after the open sum `delta`)"""
+        if x.dtype != torch.float32 or (x.dim() == 3 and x.shape[1] != 1):
+            raise ValueError("the postnorm arrangement keeps one 32-bit stream")
+        if delta is not None and not isinstance(delta, NormedSum):
+            raise ValueError("the postnorm arrangement closes a sum through a norm or nothing")
+        rows = x.view(x.shape[0], x.shape[-1])
+        joins = {} if delta is None else {"y": delta.y, "y_weight": delta.weight, "y_eps": delta.eps}
+        dtype = self.mixer.ctx.dtype
+        if dtype == torch.float32:  # (the stream itself is the input: the next sum comes after the sublayer has read it)
+            if joins:
+                ops.normed_add_norm(None, rows, None, 0.0, **joins)
+            return rows, x
+        return ops.normed_add_norm(torch.empty(rows.shape, dtype=dtype, device=x.device), rows, None, 0.0, **joins), x
+
+    def forward(self, x, delta, batch, cache):
+        h, x = self._read(x, delta)
+        y, post = self.mixer.forward(h, batch, cache), self.mixer_post_norm
+        delta = NormedSum(StreamsBlock._result(y), post.weight, post.eps)
+        if getattr(self.feed_forward, "absent", False):
+            return x, delta
+        h, x = self._read(x, delta)
+        y, post = self.feed_forward.forward(h), self.feed_forward_post_norm
+        return x, NormedSum(StreamsBlock._result(y), post.weight, post.eps)

@@ -77,13 +77,14 @@ class LayerNorm32(Norm):
 class RMSNormStreams(LayerNorm32):
     """The same over the same streams without taking the mean off: u / sqrt(mean(u^2) + eps) * w, all in 32-bit,
     rounded once.  Parameters as above, and `scalar` (True: the weight is one number for all coordinates, a tensor
-    without dimensions; default False)."""
+    without dimensions; default False), `multiplier` (the normed row is multiplied by it; default 1)."""
 
     center = False
 
     def __init__(self, spec, ctx):
         super().__init__(spec, ctx)
         self.scalar = bool(spec.get("scalar", False))
+        self.multiplier = float(spec.get("multiplier", 1.0))
 
     def param_infos(self):
         return {self.tensor: ParamInfo((), "norm")} if self.scalar else super().param_infos()
@@ -92,6 +93,8 @@ class RMSNormStreams(LayerNorm32):
         super().load(tensors)
         if self.scalar:  # (the kernels read a weight per coordinate: 4 bytes a coordinate that every row of a step shares)
             self.weight = self.weight.reshape(1).expand(self.hidden).contiguous()
+        if self.multiplier != 1.0:
+            self.weight = self.weight * self.multiplier
 
     closes_normed_sums = True  # `read_streams`, `add_norm` and `norm_rows` also take a `NormedSum` in the place of delta
 

@@ -13,7 +13,7 @@ import torch
 
 from ..ops import library as ops
 from . import (attention, attention_composed, attention_latent, block, connection, decay_attention, delta_rule, embedding,  # noqa: F401
-               experts, gate, layernorm, rmsnorm, rope, selective_scan, side_by_side, swiglu, ungated)  # (register the built-in parts)
+               experts, gate, layernorm, rmsnorm, rope, selective_scan, side_by_side, state_space, swiglu, ungated)  # (register the built-in parts)
 from .registry import (BLOCKS, CONNECTIONS, EMBEDDINGS, FEED_FORWARDS, GATES, HEADS, MIXERS, NORMS, BuildContext, DeferredNorm,
                        OpenStreams, Part)
 from .spec import ModelSpec, ParamInfo

@@ -1,6 +1,7 @@
 """Gated feed-forward: down(silu(gate(x)) * up(x)), no biases
-(src/llmserve/model/llama.py:112-120).  Parameters: hidden, intermediate, and optionally unit ("silu", or "clamped" with
-`limit`: down(g sigmoid(1.702 g) (u + 1)), g = min(gate(x), limit), u = clamp(up(x), -limit, limit)).
+(src/llmserve/model/llama.py:112-120).  Parameters: hidden, intermediate, and optionally unit ("silu"; "clamped" with
+`limit`: down(g sigmoid(1.702 g) (u + 1)), g = min(gate(x), limit), u = clamp(up(x), -limit, limit); or "gelu_tanh":
+down(gelu(gate(x)) * up(x)) with the tanh form of gelu).
 gate_proj and up_proj are stacked into one [2I, H] matrix at load, so one product feeds
 the activation.  With few bfloat16 rows that product also does the activation after it
 (ops.gemm_stream); otherwise the product and the activation are kernels of their own."""
@@ -30,9 +31,10 @@ class SwiGLU(FeedForward):
         self.names = {k: names.get(k, f"{k}_proj.weight") for k in ("gate", "up", "down")}
         self.result_dtype = torch.float32 if spec.get("result", "model") == "float32" else None
         self.unit = spec.get("unit", "silu")
-        if self.unit not in ("silu", "clamped"):
-            raise ValueError(f"unit={self.unit!r}; choose 'silu' or 'clamped'")
+        if self.unit not in ("silu", "clamped", "gelu_tanh"):
+            raise ValueError(f"unit={self.unit!r}; choose 'silu', 'clamped' or 'gelu_tanh'")
         self.limit = float(spec["limit"]) if self.unit == "clamped" else None
+        self.gelu = self.unit == "gelu_tanh"
         self.gate_up: torch.Tensor | None = None
         self.down: torch.Tensor | None = None
 
@@ -57,15 +59,15 @@ class SwiGLU(FeedForward):
                 x.resolve(None)  # nothing is left to add: the kernel norms the residual rows as they are
             elif deferred:
                 rows = x.materialize()
-            ops.gemm_decode(act, rows, self.gate_up, swiglu=True, norm=norm, limit=self.limit)  # norm before, activation after the product
+            ops.gemm_decode(act, rows, self.gate_up, swiglu=True, norm=norm, limit=self.limit, gelu=self.gelu)  # norm before, activation after the product
         else:
             if deferred:
                 rows = x.materialize()
             few = dtype == torch.bfloat16 and few_rows(m, self.gate_up) and self.intermediate % 8 == 0
             if few and ops.gemm_bf16_supported(rows, self.gate_up):
-                ops.gemm_stream(act, rows, self.gate_up, swiglu=True, limit=self.limit)  # activation in the product's epilogue
+                ops.gemm_stream(act, rows, self.gate_up, swiglu=True, limit=self.limit, gelu=self.gelu)  # activation in the product's epilogue
             else:
-                ops.silu_mul(act, linear(rows, self.gate_up), self.limit)
+                ops.silu_mul(act, linear(rows, self.gate_up), self.limit, self.gelu)
         if deferred and x.may_add_in_place and adds_residual_in_epilogue(act, self.down):
             ops.gemm_decode(None, act, self.down, residual=x.residual)  # the residual sum in the product's epilogue
             return ADDED_IN_PLACE
