@@ -26,13 +26,14 @@ first token, inter-token latency percentiles and the number of preemptions besid
 `--pages-fraction` shrinks the cache pool below what the whole workload needs, so that
 requests wait and are preempted.
 
-    python bench.py --workload designs [--design dibepel|milozen|felavik|nolavik|zotunex] [--beside llama|felavik|...] [--sizes 1b,7b] [--layers 6] [--batches 8,32] [--context 512]
+    python bench.py --workload designs [--design dibepel|milozen|felavik|nolavik|zotunex|ramolix] [--beside llama|felavik|...] [--sizes 1b,7b] [--layers 6] [--batches 8,32] [--context 512]
 
 puts the Dibepel design (or, with `--design milozen`, the Milozen design: latent attention, experts, two streams; with
 `--design felavik`, the Felavik design: linear attention with a decay per head, gated softmax attention, experts in groups;
 with `--design nolavik`, the Nolavik design: latent attention, the gated delta rule, sink attention beside a selective scan,
 experts with a shared expert, a looped layer; with `--design zotunex`, the Zotunex design: attention whose values are its
-keys, latent attention with sinks, squared-relu and expert feed-forwards)
+keys, latent attention with sinks, squared-relu and expert feed-forwards; with `--design ramolix`, the Ramolix design:
+state-space layers, windowed attention whose values are its keys, latent attention over shared latents, gelu feed-forwards)
 beside the Llama decoder at equal layer sizes (width, heads, key/value heads, head size,
 feed-forward, vocabulary, layers; random weights): prefill tokens a second for one prompt of 2,048 tokens in one
 step, and decoded tokens a second at the given batch sizes behind `--context` tokens, both through the step
@@ -322,6 +323,32 @@ def zotunex_config(size: dict, layers: int, experts: int = 8, top: int = 2) -> d
             "layers": entries}
 
 
+def ramolix_config(size: dict, layers: int, window: int = 1024, states: int = 128, head: int = 64) -> dict:
+    """In turn: windowed attention of the Llama shape's heads and key/value heads whose values are the keys (all of a head
+    turned, stretched frequencies), latent attention (as many heads, values of the head size, a latent of four head sizes;
+    from the second on every such layer reads the first one's latents), and two state-space layers twice as wide as the model
+    (heads of 64 columns, 128 states, 8 groups, 4 taps); the dense feed-forward of the Llama shape, gated by gelu."""
+    dim, heads, width = size["dim"], size["heads"], size["width"]
+    mlp = {"kind": "dense", "ff": size["ff"]}
+    entries = []
+    for i in range(layers):
+        if i % 4 == 0:
+            entry = {"type": "attention", "mixer": {
+                "heads": heads, "kv_heads": size["kv_heads"], "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": window},
+                "rot": {"base": 500000.0, "dims": dim, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}}
+        elif i % 4 == 1:
+            entry = {"type": "latent_attention", "mixer": {"heads": heads, "dim": dim, "vdim": dim, "kv_rank": 4 * dim,
+                                                           "scale": dim ** -0.5}}
+            if i > 1:
+                entry["mixer"]["kv_from"] = 1
+        else:
+            entry = {"type": "mamba2", "mixer": {"heads": 2 * width // head, "vdim": head, "state": states, "groups": 8, "conv": 4,
+                                                 "norm_groups": 8}}
+        entries.append(dict(entry, mlp=mlp))
+    return {"architecture": "Ramolix", "vocab": size["vocab"], "width": width, "embedding": {"scale": width ** 0.5},
+            "norm": {"eps": 1e-5}, "residual_mult": 0.5, "layers": entries}
+
+
 def llama_config(size: dict, layers: int, positions: int) -> dict:
     return dict(architectures=["LlamaForCausalLM"], model_type="llama", vocab_size=size["vocab"], hidden_size=size["width"],
                 intermediate_size=size["ff"], num_hidden_layers=layers, num_attention_heads=size["heads"],
@@ -397,7 +424,7 @@ def designs(args) -> int:
     table = {}
     design = args.design
     makers = {"dibepel": dibepel_config, "milozen": milozen_config, "felavik": felavik_config, "nolavik": nolavik_config,
-              "zotunex": zotunex_config}
+              "zotunex": zotunex_config, "ramolix": ramolix_config}
     make, beside = makers[design], args.beside
     if beside == design:
         raise SystemExit("--beside names the design itself")
@@ -542,9 +569,9 @@ def main() -> int:
                     help="run one phase only (for profiles; the line then holds zeros for the other); gemv: the "
                          "decode products alone, each over copies of its weight that do not fit the caches")
     ap.add_argument("--workload", choices=["steps", "serve", "designs"], default="steps")
-    ap.add_argument("--design", choices=["dibepel", "milozen", "felavik", "nolavik", "zotunex"], default="dibepel",
+    ap.add_argument("--design", choices=["dibepel", "milozen", "felavik", "nolavik", "zotunex", "ramolix"], default="dibepel",
                     help="designs: which design is measured")
-    ap.add_argument("--beside", choices=["llama", "dibepel", "milozen", "felavik", "nolavik", "zotunex"], default="llama",
+    ap.add_argument("--beside", choices=["llama", "dibepel", "milozen", "felavik", "nolavik", "zotunex", "ramolix"], default="llama",
                     help="designs: the model it stands beside, at equal layer sizes")
     ap.add_argument("--sizes", default="1b,7b", help="designs: layer sizes to compare at")
     ap.add_argument("--batches", default="8,32", help="designs: decode batch sizes")

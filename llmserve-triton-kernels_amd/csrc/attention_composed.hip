@@ -15,7 +15,8 @@
 //                 the norm; q is then multiplied by 1 + coef * ln(floor((p + 1) / every) + 1) at position p (every 0: no
 //                 factor) and by a number per head (q_scale); all in 32-bit, rounded once, into the query rows and the
 //                 cache slots.  `v_from_k`: the values are the keys as projected, before norm and rotation.  `joint`: the
-//                 norm is over all heads of q at once, and over all of k, with a weight per number ([heads * dk]).
+//                 norm is over all heads of q at once, and over all of k, with a weight per number ([heads * dk]); a bias
+//                 [columns] may be added to the projection first.
 //   attend        one workgroup per new token, all heads.  Score heads s = h * maps + m (maps = 2: two score maps
 //                 per query head over the same values); s reads key head (h / (H / G)) * maps + m, values come from
 //                 value head h / (H / G).  A query at position i sees the key j <= i if
@@ -127,6 +128,7 @@ struct HeadStoreArgs {
     int norm_first;  // the norm comes before the rotation
     int v_from_k;    // values are the keys as projected (v_heads = k_heads, dv = dk; proj holds no values)
     int joint;       // one norm over all heads of q, one over all heads of k; the weights hold heads * dk numbers
+    const float* bias;  // of every column of proj, or null (with `joint` only)
 };
 
 __device__ __forceinline__ float2 head_angle(const HeadStoreArgs& a, int n, float position, int i) {  // (sine, cosine)
@@ -350,92 +352,156 @@ __device__ __forceinline__ bool head_slot(const HeadStoreArgs& a, int n, int& pa
     return slot >= 0;
 }
 
-// values of 16 tokens of one value head, through LDS into a page's transposed rows
+// values of 16 tokens of one value head, through LDS into a page's transposed rows; 8 tokens that lie side by side in a page
+// leave as one 16-byte piece of a dimension (bfloat16)
 template <typename T>
-__device__ __forceinline__ void store_values(T* __restrict__ v_pool, const HeadStoreArgs& a, int n0, int head, float* tile, long long* place) {
+__device__ __forceinline__ void store_values(T* __restrict__ v_pool, const HeadStoreArgs& a, int n0, int head, float* tile,
+                                             long long* place, int* side_by_side) {
     const int tid = threadIdx.x, dv = a.dv, pitch = dv + 1;
     if (tid < HS_TOKENS) {
         int page, off;
         const bool in = n0 + tid < a.n_tokens && head_slot(a, n0 + tid, page, off);
         place[tid] = in ? ((long long)page * a.v_heads + head) * dv * a.block_size + off : -1;
     }
-    const float* src = a.proj + (a.v_from_k ? (size_t)(a.q_heads + head) * a.dk : (size_t)(a.q_heads + a.k_heads) * a.dk + (size_t)head * dv);
-    for (int i = tid; i < HS_TOKENS * dv; i += HS_THREADS) {
-        const int t = i / dv, d = i - t * dv;
-        if (n0 + t < a.n_tokens) tile[t * pitch + d] = src[(size_t)(n0 + t) * a.proj_stride + d];
+    const int col = a.v_from_k ? (a.q_heads + head) * a.dk : (a.q_heads + a.k_heads) * a.dk + head * dv;
+    if (dv % 4 == 0) {  // (the rows of proj and its columns are at multiples of 16 bytes here)
+        for (int i = tid; i < HS_TOKENS * (dv / 4); i += HS_THREADS) {
+            const int t = i / (dv / 4), d = 4 * (i - t * (dv / 4));
+            if (n0 + t >= a.n_tokens) continue;
+            float4 v = *reinterpret_cast<const float4*>(a.proj + (size_t)(n0 + t) * a.proj_stride + col + d);
+            if (a.bias) {
+                const float4 b = *reinterpret_cast<const float4*>(a.bias + col + d);
+                v.x += b.x, v.y += b.y, v.z += b.z, v.w += b.w;
+            }
+            float* at = tile + t * pitch + d;
+            at[0] = v.x, at[1] = v.y, at[2] = v.z, at[3] = v.w;
+        }
+    } else {
+        for (int i = tid; i < HS_TOKENS * dv; i += HS_THREADS) {
+            const int t = i / dv, d = i - t * dv;
+            if (n0 + t < a.n_tokens)
+                tile[t * pitch + d] = a.proj[(size_t)(n0 + t) * a.proj_stride + col + d] + (a.bias ? a.bias[col + d] : 0.f);
+        }
     }
     __syncthreads();
+    if constexpr (sizeof(T) == 2) {
+        if (tid < 2) {
+            bool joined = place[8 * tid] >= 0 && place[8 * tid] % 8 == 0 && a.block_size % 8 == 0 && ((uintptr_t)v_pool % 16) == 0;
+            for (int t = 1; t < 8; ++t) joined = joined && place[8 * tid + t] == place[8 * tid] + t;
+            side_by_side[tid] = joined;
+        }
+        __syncthreads();
+        if (side_by_side[0] && side_by_side[1]) {
+            for (int i = tid; i < 2 * dv; i += HS_THREADS) {
+                const int g = i & 1, d = i >> 1;
+                const float* at = tile + 8 * g * pitch + d;
+                uint32_t w[4];
+#pragma unroll
+                for (int k = 0; k < 4; ++k) w[k] = pack_bf16x2(at[2 * k * pitch], at[(2 * k + 1) * pitch]);
+                *reinterpret_cast<uint4*>(v_pool + place[8 * g] + (long long)d * a.block_size) = make_uint4(w[0], w[1], w[2], w[3]);
+            }
+            return;
+        }
+    }
     for (int i = tid; i < HS_TOKENS * dv; i += HS_THREADS) {
         const int t = i % HS_TOKENS, d = i / HS_TOKENS;
         if (place[t] >= 0) v_pool[place[t] + (long long)d * a.block_size] = from_f32<T>(tile[t * pitch + d]);
     }
 }
 
-// Heads of 16, 32, 64, 128 or 256 numbers, rows of q and k of up to 256 V numbers: a wave takes a row (the q or the k of a
-// token) and keeps it in registers, V pieces of 256 numbers of whole heads, so a row costs one trip to memory and no
-// barrier, and a pair of the rotation lies in two lanes of one piece.  The first `v_blocks` workgroups store values.
-template <typename T, int V>
+// Heads of 16, 32, 64, 128 or 256 numbers, rows of q and k of up to 4 LANES V numbers: LANES lanes (a wave or a workgroup)
+// take a row (the q or the k of a token) and keep it in registers, V pieces of 16 bytes a lane, so a row costs one trip to
+// memory, and since the 256 numbers of a wave's piece are whole heads, a pair of the rotation lies in two of its lanes.  ROWS
+// tokens one after the other, the next one asked for before the present one is worked on; weights and biases stay in
+// registers.  The first `v_blocks` workgroups store values.
+template <typename T, int LANES, int V, int ROWS>
 __global__ __launch_bounds__(HS_THREADS) void joint_rows_kernel(T* __restrict__ q_out, T* __restrict__ k_pool,
                                                                 T* __restrict__ v_pool, HeadStoreArgs a, int v_blocks) {
     __shared__ float tile[HS_TOKENS * (HS_MAX_DIM + 1)];
     __shared__ long long place[HS_TOKENS];
+    __shared__ float red[16];
     if ((int)blockIdx.x < v_blocks) {
-        store_values<T>(v_pool, a, ((int)blockIdx.x / a.v_heads) * HS_TOKENS, (int)blockIdx.x % a.v_heads, tile, place);
+        store_values<T>(v_pool, a, ((int)blockIdx.x / a.v_heads) * HS_TOKENS, (int)blockIdx.x % a.v_heads, tile, place, (int*)red);
         return;
     }
-    const int lane = threadIdx.x % LLMS_WAVE, dk = a.dk;
-    const int r = ((int)blockIdx.x - v_blocks) * (HS_THREADS / LLMS_WAVE) + threadIdx.x / LLMS_WAVE;
-    const int n = r >> 1;
-    const bool is_q = (r & 1) == 0;
-    if (n >= a.n_tokens) return;
-    int page = 0, off = 0;
-    if (!is_q && !head_slot(a, n, page, off)) return;
-    const int width = (is_q ? a.q_heads : a.k_heads) * dk;
-    const float* src = a.proj + (size_t)n * a.proj_stride + (is_q ? 0 : (size_t)a.q_heads * dk);
+    const int lane = threadIdx.x % LLMS_WAVE, at = threadIdx.x % LANES, dk = a.dk;
+    const int item = ((int)blockIdx.x - v_blocks) * (HS_THREADS / LANES) + threadIdx.x / LANES;
+    const bool is_q = (item & 1) == 0;
+    const int n0 = (item >> 1) * ROWS;
+    if (n0 >= a.n_tokens || (!is_q && !a.slots)) return;  // (whole waves; with LANES = 256 the whole workgroup)
+    const int width = (is_q ? a.q_heads : a.k_heads) * dk, col = is_q ? 0 : a.q_heads * dk;
     const float* w = is_q ? a.q_norm : a.k_norm;
-    float4 x[V], wv[V];
-    float ss = 0.f;
-#pragma unroll
-    for (int v = 0; v < V; ++v) {
-        const int c = 4 * (v * LLMS_WAVE + lane);
-        const float4 one = make_float4(1.f, 1.f, 1.f, 1.f);
-        x[v] = c < width ? *reinterpret_cast<const float4*>(src + c) : make_float4(0.f, 0.f, 0.f, 0.f);
-        wv[v] = (w && c < width) ? *reinterpret_cast<const float4*>(w + c) : one;
-    }
-    // the lane's angles are the same in every piece: a piece holds whole heads
     const int lph = dk >> 2, li = lane & (lph - 1), half = a.rot_dims >> 1;
     const int hl = half >> 2;
     const bool turns = li < 2 * hl, low = li < hl;
-    float2 sc[4];
-#pragma unroll
-    for (int e = 0; e < 4; ++e)
-        sc[e] = turns ? a.angles[(size_t)n * half + 4 * (low ? li : li - hl) + e] : make_float2(0.f, 1.f);
-#pragma unroll
-    for (int v = 0; v < V; ++v) ss += (x[v].x * x[v].x + x[v].y * x[v].y) + (x[v].z * x[v].z + x[v].w * x[v].w);
-    const float mul = 1.f / sqrtf(wave_sum(ss) / (float)width + a.eps);
     const int partner = turns ? (low ? lane + hl : lane - hl) : lane;
+    struct Row {
+        float4 x[V];
+        float2 sc[4];  // (the lane's angles are the same in every piece: a piece holds whole heads)
+        int slot;
+    };
+    auto fetch = [&](Row& r, int n) {
+        const float* src = a.proj + (size_t)n * a.proj_stride + col;
+        r.slot = is_q ? 0 : a.slots[n];
+#pragma unroll
+        for (int v = 0; v < V; ++v) {
+            const int c = 4 * (v * LANES + at);
+            r.x[v] = c < width ? *reinterpret_cast<const float4*>(src + c) : make_float4(0.f, 0.f, 0.f, 0.f);
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+            r.sc[e] = turns ? a.angles[(size_t)n * half + 4 * (low ? li : li - hl) + e] : make_float2(0.f, 1.f);
+    };
+    float4 wv[V], bv[V];
+    Row row;
+    fetch(row, n0);
 #pragma unroll
     for (int v = 0; v < V; ++v) {
-        const int c = 4 * (v * LLMS_WAVE + lane);
-        float y[4] = {x[v].x * mul * wv[v].x, x[v].y * mul * wv[v].y, x[v].z * mul * wv[v].z, x[v].w * mul * wv[v].w};
-        if (hl > 0) {
+        const int c = 4 * (v * LANES + at);
+        const float4 one = make_float4(1.f, 1.f, 1.f, 1.f), zero = make_float4(0.f, 0.f, 0.f, 0.f);
+        wv[v] = (w && c < width) ? *reinterpret_cast<const float4*>(w + c) : one;
+        bv[v] = (a.bias && c < width) ? *reinterpret_cast<const float4*>(a.bias + col + c) : zero;
+    }
 #pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const float other = __shfl(y[e], partner, LLMS_WAVE);
-                const float2 t = low ? rotate_pair(y[e], other, sc[e].y, sc[e].x) : rotate_pair(other, y[e], sc[e].y, sc[e].x);
-                if (turns) y[e] = low ? t.x : t.y;
+    for (int i = 0; i < ROWS; ++i) {
+        const int n = n0 + i;
+        if (n >= a.n_tokens) break;
+        Row next;
+        if (i + 1 < ROWS) fetch(next, min(n + 1, a.n_tokens - 1));
+        float ss = 0.f;
+#pragma unroll
+        for (int v = 0; v < V; ++v) {
+            float4& x = row.x[v];
+            x.x += bv[v].x, x.y += bv[v].y, x.z += bv[v].z, x.w += bv[v].w;
+            ss += (x.x * x.x + x.y * x.y) + (x.z * x.z + x.w * x.w);
+        }
+        const float mul = 1.f / sqrtf((LANES == LLMS_WAVE ? wave_sum(ss) : block_sum(ss, red)) / (float)width + a.eps);
+        const int page = row.slot / a.block_size, off = row.slot - page * a.block_size;
+#pragma unroll
+        for (int v = 0; v < V; ++v) {
+            const int c = 4 * (v * LANES + at);
+            const float4 x = row.x[v];
+            float y[4] = {x.x * mul * wv[v].x, x.y * mul * wv[v].y, x.z * mul * wv[v].z, x.w * mul * wv[v].w};
+            if (hl > 0) {
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    const float other = __shfl(y[e], partner, LLMS_WAVE);
+                    const float2 t = low ? rotate_pair(y[e], other, row.sc[e].y, row.sc[e].x) : rotate_pair(other, y[e], row.sc[e].y, row.sc[e].x);
+                    if (turns) y[e] = low ? t.x : t.y;
+                }
+            }
+            if (c >= width) continue;
+            const int head = c / dk, d = c - head * dk;
+            if (is_q) {
+                const float factor = query_factor(a, n, head);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) y[e] *= factor;
+                store4<T>(q_out + (size_t)n * a.q_stride + c, y);
+            } else if (row.slot >= 0) {
+                store4<T>(k_pool + (((size_t)page * a.k_heads + head) * a.block_size + off) * dk + d, y);
             }
         }
-        if (c >= width) continue;
-        const int head = c / dk, d = c - head * dk;
-        if (is_q) {
-            const float factor = query_factor(a, n, head);
-#pragma unroll
-            for (int e = 0; e < 4; ++e) y[e] *= factor;
-            store4<T>(q_out + (size_t)n * a.q_stride + c, y);
-        } else {
-            store4<T>(k_pool + (((size_t)page * a.k_heads + head) * a.block_size + off) * dk + d, y);
-        }
+        if (i + 1 < ROWS) row = next;
     }
 }
 
@@ -452,17 +518,18 @@ __global__ __launch_bounds__(HS_THREADS) void joint_store_kernel(T* __restrict__
     if (role >= 2) {
         const int head = role - 2;
         const float* src = row + (a.v_from_k ? (size_t)(a.q_heads + head) * dk : (size_t)(a.q_heads + a.k_heads) * dk + (size_t)head * dv);
+        const float* bias = a.bias ? a.bias + (src - row) : nullptr;
         for (int d = threadIdx.x; d < dv; d += HS_THREADS)
-            v_pool[(((size_t)page * a.v_heads + head) * dv + d) * a.block_size + off] = from_f32<T>(src[d]);
+            v_pool[(((size_t)page * a.v_heads + head) * dv + d) * a.block_size + off] = from_f32<T>(src[d] + (bias ? bias[d] : 0.f));
         return;
     }
     const bool is_q = role == 0;
-    const int width = (is_q ? a.q_heads : a.k_heads) * dk;
-    const float* src = row + (is_q ? 0 : (size_t)a.q_heads * dk);
+    const int width = (is_q ? a.q_heads : a.k_heads) * dk, col = is_q ? 0 : a.q_heads * dk;
+    const float* src = row + col;
     const float* w = is_q ? a.q_norm : a.k_norm;
     float ss = 0.f;
     for (int i = threadIdx.x; i < width; i += HS_THREADS) {
-        const float x = src[i];
+        const float x = src[i] + (a.bias ? a.bias[col + i] : 0.f);
         joint_row[i] = w ? x * w[i] : x;
         ss = fmaf(x, x, ss);
     }
@@ -480,20 +547,31 @@ __global__ __launch_bounds__(HS_THREADS) void joint_store_kernel(T* __restrict__
 template <typename T>
 static int launch_joint_store(T* q_out, T* k_pool, T* v_pool, const HeadStoreArgs& a, hipStream_t stream) {
     const int half = a.rot_dims / 2, longest = (a.q_heads > a.k_heads ? a.q_heads : a.k_heads) * a.dk;
-    const bool rows = (a.dk == 16 || a.dk == 32 || a.dk == 64 || a.dk == 128 || a.dk == 256) && longest <= 4096 && a.dv <= HS_MAX_DIM &&
+    const bool rows = (a.dk == 16 || a.dk == 32 || a.dk == 64 || a.dk == 128 || a.dk == 256) && longest <= 8192 && a.dv <= HS_MAX_DIM &&
                       a.proj_stride % 4 == 0 && a.q_stride % 4 == 0 && ((uintptr_t)a.proj % 16) == 0 && ((uintptr_t)q_out % 16) == 0 &&
-                      (!k_pool || ((uintptr_t)k_pool % 16) == 0) && ((uintptr_t)a.q_norm % 16) == 0 && ((uintptr_t)a.k_norm % 16) == 0 &&
+                      (!k_pool || ((uintptr_t)k_pool % 16) == 0) && ((uintptr_t)a.q_norm % 16) == 0 && ((uintptr_t)a.k_norm % 16) == 0 && ((uintptr_t)a.bias % 16) == 0 &&
                       (a.rot_dims == 0 || (a.angles && !a.neighbours && half % 4 == 0));
     if (rows) {
         const int v_blocks = a.slots ? (a.n_tokens + HS_TOKENS - 1) / HS_TOKENS * a.v_heads : 0;
-        const int per = HS_THREADS / LLMS_WAVE;
         LLMS_REQUIRE(2ll * a.n_tokens + v_blocks < (1ll << 30), "norm_store: too many tokens for one launch");
-        const unsigned grid = (unsigned)(v_blocks + (2 * a.n_tokens + per - 1) / per);
-        if (longest <= 256) joint_rows_kernel<T, 1><<<grid, HS_THREADS, 0, stream>>>(q_out, k_pool, v_pool, a, v_blocks);
-        else if (longest <= 512) joint_rows_kernel<T, 2><<<grid, HS_THREADS, 0, stream>>>(q_out, k_pool, v_pool, a, v_blocks);
-        else if (longest <= 1024) joint_rows_kernel<T, 4><<<grid, HS_THREADS, 0, stream>>>(q_out, k_pool, v_pool, a, v_blocks);
-        else if (longest <= 2048) joint_rows_kernel<T, 8><<<grid, HS_THREADS, 0, stream>>>(q_out, k_pool, v_pool, a, v_blocks);
-        else joint_rows_kernel<T, 16><<<grid, HS_THREADS, 0, stream>>>(q_out, k_pool, v_pool, a, v_blocks);
+        // many tokens: a wave (of long rows a workgroup) walks two rows; few: the lanes of a workgroup share a row out
+#define JOINT_GO(LANES, V, ROWS)                                                                                          \
+    do {                                                                                                                  \
+        const int per = HS_THREADS / LANES, items = 2 * ((a.n_tokens + ROWS - 1) / ROWS);                                 \
+        joint_rows_kernel<T, LANES, V, ROWS><<<(unsigned)(v_blocks + (items + per - 1) / per), HS_THREADS, 0, stream>>>(   \
+            q_out, k_pool, v_pool, a, v_blocks);                                                                          \
+    } while (0)
+        const bool many = a.n_tokens >= 512;
+        if (longest <= 256) JOINT_GO(64, 1, 1);
+        else if (longest <= 512) JOINT_GO(64, 2, 1);
+        else if (longest <= 1024 && many) JOINT_GO(64, 4, 2);
+        else if (longest <= 1024) JOINT_GO(256, 1, 1);
+        else if (longest <= 2048 && many) JOINT_GO(64, 8, 2);
+        else if (longest <= 2048) JOINT_GO(256, 2, 1);
+        else if (longest <= 4096 && many) JOINT_GO(256, 4, 2);
+        else if (longest <= 4096) JOINT_GO(256, 4, 1);
+        else JOINT_GO(256, 8, 1);
+#undef JOINT_GO
         LLMS_LAUNCH_CHECK();
     }
     const size_t lds = (size_t)longest * sizeof(float);
@@ -765,7 +843,7 @@ int llms_norm_store(int dtype, void* q_out, int q_stride, const float* proj, int
                     const float* k_norm, float eps, float temp_coef, int temp_every, const int* positions, const int* slots,
                     void* k_pool, void* v_pool, int n_tokens, int q_heads, int k_heads, int dk, int v_heads, int dv,
                     int block_size, const float* freq, const float* angles, int rot_dims, int unit_norm, int neighbours,
-                    int norm_first, const float* q_scale, int v_from_k, int joint, hipStream_t stream) {
+                    int norm_first, const float* q_scale, int v_from_k, int joint, const float* bias, hipStream_t stream) {
     LLMS_REQUIRE(n_tokens > 0 && q_heads > 0 && k_heads >= 0 && v_heads >= 0 && dk > 0 && dv > 0, "norm_store: sizes must be positive");
     LLMS_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= dk && (rot_dims == 0 || angles || (freq && positions)),
                  "norm_store: an even number of turned dimensions within a head, with angles or frequencies and positions");
@@ -780,7 +858,8 @@ int llms_norm_store(int dtype, void* q_out, int q_stride, const float* proj, int
     a.eps = eps, a.temp_coef = temp_coef, a.temp_every = temp_every;
     a.n_tokens = n_tokens, a.q_heads = q_heads, a.k_heads = k_heads, a.dk = dk, a.v_heads = v_heads, a.dv = dv;
     a.block_size = block_size > 0 ? block_size : 1, a.rot_dims = rot_dims;
-    a.unit_norm = unit_norm, a.neighbours = neighbours, a.norm_first = norm_first, a.v_from_k = v_from_k, a.joint = joint;
+    a.unit_norm = unit_norm, a.neighbours = neighbours, a.norm_first = norm_first, a.v_from_k = v_from_k, a.joint = joint, a.bias = bias;
+    LLMS_REQUIRE(!bias || joint, "norm_store: a bias goes with one norm over all heads");
     LLMS_REQUIRE(!joint || norm_first || rot_dims == 0, "norm_store: one norm over all heads comes before the rotation");
     LLMS_REQUIRE(!joint || rot_dims == 0 || positions, "norm_store: a rotation needs the positions");
     if (dtype == 0) return launch_norm_store<float>((float*)q_out, (float*)k_pool, (float*)v_pool, a, stream);

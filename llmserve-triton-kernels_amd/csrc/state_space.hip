@@ -56,7 +56,16 @@ struct SpaceArgs {
     const int* context_lens;
 };
 
+// SiLU behind the convolution: 32-bit, or, where its result is rounded to bfloat16 anyway, by the hardware's exponential and
+// reciprocal (both within an ulp of 32-bit)
+template <typename T>
+__device__ __forceinline__ float sp_silu(float x) {
+    if constexpr (sizeof(T) == 2) return x * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.44269504f * x));
+    else return rc_silu(x);
+}
+
 // channel c of the convolution at row `row` (position pos) of a portion that starts at first_row (position first_pos)
+template <typename T>
 __device__ __forceinline__ float sp_conv(const SpaceArgs& a, const float* __restrict__ ring, int first_row, int first_pos, int pos, int c) {
     float y = a.bias[c];
     for (int j = 0; j < a.taps; ++j) {
@@ -66,7 +75,7 @@ __device__ __forceinline__ float sp_conv(const SpaceArgs& a, const float* __rest
         else if (at >= 0) v = ring[(size_t)(at % (a.taps - 1)) * a.channels + c];
         y = fmaf(a.taps_w[(size_t)c * a.taps + j], v, y);
     }
-    return rc_silu(y);
+    return sp_silu<T>(y);
 }
 
 // ------------------------------------------------------------------------------------------- token by token
@@ -103,7 +112,7 @@ __global__ __launch_bounds__(SP_THREADS) void space_scan_kernel(float* __restric
         float* row = sp_rows + (t & 1) * pitch;  // [x of the 16 columns | B | C | dt, decay]
         for (int i = threadIdx.x; i < need; i += SP_THREADS) {
             const int c = i < 16 ? h * a.P + min(p0 + i, a.P - 1) : inner + (i - 16 < N ? g * N + i - 16 : (a.groups + g) * N + i - 16 - N);
-            row[i] = round_to<T>(sp_conv(a, ring, first_row, first_pos, first_pos + t, c));
+            row[i] = round_to<T>(sp_conv<T>(a, ring, first_row, first_pos, first_pos + t, c));
         }
         if (threadIdx.x == SP_THREADS - 1) {
             const float dt = rc_softplus(a.u[(size_t)(first_row + t) * a.u_ld + a.dt_col + h] + dt_bias);
@@ -246,7 +255,7 @@ __global__ __launch_bounds__(SP_THREADS) void space_prepare_kernel(const SpaceAr
         float s = bias;
 #pragma unroll
         for (int k = 0; k < TAPS; ++k) s = fmaf(tap[k], in[i + k], s);
-        out[i] = t0 + i < count ? rc_silu(s) : 0.f;
+        out[i] = t0 + i < count ? sp_silu<bf16>(s) : 0.f;
     }
     uint32_t packed[8];
 #pragma unroll
@@ -264,7 +273,8 @@ __global__ __launch_bounds__(SP_THREADS) void space_prepare_kernel(const SpaceAr
     }
 }
 
-// grid (runs of the longest portion, heads x slabs + groups, requests)
+// grid (runs of the longest portion, groups + heads x slabs, requests)
+#define SP_STATE_STEPS 8  // steps of 32 states
 __global__ __launch_bounds__(SP_THREADS) void space_sums_kernel(const SpaceArgs a, const RunSpace w, int slabs) {
     __shared__ float2 logs[SP_RUN];
     __shared__ float weight[SP_RUN];
@@ -276,29 +286,47 @@ __global__ __launch_bounds__(SP_THREADS) void space_sums_kernel(const SpaceArgs 
     const int inner = a.heads * P, gn = a.groups * N;
     const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
     const bf16x8 none = __builtin_bit_cast(bf16x8, make_uint4(0, 0, 0, 0));
-    if ((int)blockIdx.y >= a.heads * slabs) {  // B_s . C_t of a group: wave i takes the token tiles i and 7 - i
-        const int g = blockIdx.y - a.heads * slabs;
-        const bf16* rows = w.bc + (size_t)(first_row + j * SP_RUN) * (2 * gn) + g * N;
+    if ((int)blockIdx.y < a.groups) {  // B_s . C_t of a group: wave i takes the token tiles i and 7 - i
+        const int g = blockIdx.y;
+        const bf16* rows = w.bc + (size_t)(first_row + j * SP_RUN) * (2 * gn) + g * N + 8 * hi;
         float* dst = w.scores + ((size_t)place * a.groups + g) * (SP_SCORE_TILES * 256);
         for (int half = 0; half < 2; ++half) {
             const int tt = half ? SP_TILES - 1 - wave : wave;
             if (16 * tt >= n) continue;
-            const int t = 16 * tt + lo;
+            const bf16* ct_at = rows + (size_t)min(16 * tt + lo, n - 1) * (2 * gn) + gn;  // (columns behind the last token are not read)
+            bf16x8 ct[SP_STATE_STEPS];
+#pragma unroll
+            for (int k = 0; k < SP_STATE_STEPS; ++k) {
+                if (32 * k >= N) break;
+                ct[k] = 32 * k + 8 * hi < N ? *reinterpret_cast<const bf16x8*>(ct_at + 32 * k) : none;
+            }
             for (int st = 0; st <= tt; ++st) {
-                const int s = 16 * st + lo;
+                const bf16* bs_at = rows + (size_t)min(16 * st + lo, n - 1) * (2 * gn);
+                bf16x8 bs[SP_STATE_STEPS];
+#pragma unroll
+                for (int k = 0; k < SP_STATE_STEPS; ++k) {
+                    if (32 * k >= N) break;
+                    bs[k] = 32 * k + 8 * hi < N ? *reinterpret_cast<const bf16x8*>(bs_at + 32 * k) : none;
+                }
                 f32x4 acc = zero;
-                for (int k0 = 8 * hi; k0 - 8 * hi < N; k0 += 32) {
-                    const bf16x8 bs = (s < n && k0 < N) ? *reinterpret_cast<const bf16x8*>(rows + (size_t)s * (2 * gn) + k0) : none;
-                    const bf16x8 ct = (t < n && k0 < N) ? *reinterpret_cast<const bf16x8*>(rows + (size_t)t * (2 * gn) + gn + k0) : none;
-                    acc = sp_mfma(bs, ct, acc);
+#pragma unroll
+                for (int k = 0; k < SP_STATE_STEPS; ++k) {
+                    if (32 * k >= N) break;
+                    acc = sp_mfma(bs[k], ct[k], acc);
                 }
                 *reinterpret_cast<f32x4*>(dst + ((size_t)(tt * (tt + 1) / 2 + st) * LLMS_WAVE + lane) * 4) = acc;
             }
         }
         return;
     }
-    const int h = blockIdx.y / slabs, c0 = (blockIdx.y % slabs) * SP_SLAB;
+    const int h = (blockIdx.y - a.groups) / slabs, c0 = ((blockIdx.y - a.groups) % slabs) * SP_SLAB;
     const size_t head_at = (size_t)place * a.heads + h;
+    const int p = c0 + 16 * wave, g = h / (a.heads / a.groups);
+    // the wave's columns of x are asked for before the weights are known
+    const bf16* xt = w.xbt + ((size_t)place * (inner + gn) + h * P + min(p, P - 16) + lo) * SP_RUN + 8 * hi;
+    uint4 xraw[SP_RUN / 32];
+#pragma unroll
+    for (int k = 0; k < SP_RUN / 32; ++k) xraw[k] = *reinterpret_cast<const uint4*>(xt + 32 * k);
     if (wave == 0) {  // L_t: two tokens a lane, summed in 64-bit
         const float2 dt = *reinterpret_cast<const float2*>(w.dt + head_at * SP_RUN + 2 * lane);
         const double rate = (double)expf(a.a_log[h]);
@@ -323,30 +351,35 @@ __global__ __launch_bounds__(SP_THREADS) void space_sums_kernel(const SpaceArgs 
         }
     }
     __syncthreads();
-    const int p = c0 + 16 * wave;
     if (p >= P) return;
-    const int g = h / (a.heads / a.groups);
-    const bf16* xt = w.xbt + ((size_t)place * (inner + gn) + h * P + p + lo) * SP_RUN;
-    const bf16* bt = w.xbt + ((size_t)place * (inner + gn) + inner + g * N + lo) * SP_RUN;
+    const bf16* bt = w.xbt + ((size_t)place * (inner + gn) + inner + g * N + lo) * SP_RUN + 8 * hi;
     float* dst = w.sums + (head_at * P + p + lo) * N + 4 * hi;
     for (int n0 = 0; n0 < N; n0 += 128) {
         f32x4 acc[8];
 #pragma unroll
         for (int i = 0; i < 8; ++i) acc[i] = zero;
-        for (int t = 8 * hi; t - 8 * hi < n; t += 32) {
-            const uint4 raw = *reinterpret_cast<const uint4*>(xt + t);
-            const uint32_t xw[4] = {raw.x, raw.y, raw.z, raw.w};
+#pragma unroll
+        for (int k = 0; k < SP_RUN / 32; ++k) {
+            if (32 * k >= n) break;
+            bf16x8 bs[8];
+#pragma unroll
+            for (int i = 0; i < 8; ++i) {
+                if (n0 + 16 * i >= N) break;
+                bs[i] = *reinterpret_cast<const bf16x8*>(bt + (size_t)(n0 + 16 * i) * SP_RUN + 32 * k);
+            }
+            const uint32_t xw[4] = {xraw[k].x, xraw[k].y, xraw[k].z, xraw[k].w};
             float v[8];
 #pragma unroll
-            for (int i = 0; i < 4; ++i) v[2 * i] = sp_lo(xw[i]) * weight[t + 2 * i], v[2 * i + 1] = sp_hi(xw[i]) * weight[t + 2 * i + 1];
+            for (int i = 0; i < 4; ++i) {
+                const int t = 32 * k + 8 * hi + 2 * i;
+                v[2 * i] = sp_lo(xw[i]) * weight[t], v[2 * i + 1] = sp_hi(xw[i]) * weight[t + 1];
+            }
             const Terms x = sp_split(v);
 #pragma unroll
             for (int i = 0; i < 8; ++i) {
-                if (n0 + 16 * i < N) {
-                    const bf16x8 bs = *reinterpret_cast<const bf16x8*>(bt + (size_t)(n0 + 16 * i) * SP_RUN + t);
+                if (n0 + 16 * i >= N) break;
 #pragma unroll
-                    for (int k = 2; k >= 0; --k) acc[i] = sp_mfma(bs, x.t[k], acc[i]);
-                }
+                for (int k3 = 2; k3 >= 0; --k3) acc[i] = sp_mfma(bs[i], x.t[k3], acc[i]);
             }
         }
 #pragma unroll
@@ -665,7 +698,7 @@ int llms_space_runs(float* y, int y_ld, const float* u, int u_ld, int col, int d
     LLMS_REQUIRE(grid_p.y <= 65535, "space_runs: too many channels");
     if (taps <= 4) space_prepare_kernel<4><<<grid_p, SP_THREADS, 0, stream>>>(a, w);
     else space_prepare_kernel<SP_TAPS_MAX><<<grid_p, SP_THREADS, 0, stream>>>(a, w);
-    space_sums_kernel<<<dim3(runs, heads * slabs + groups, n_seqs), SP_THREADS, 0, stream>>>(a, w, slabs);
+    space_sums_kernel<<<dim3(runs, groups + heads * slabs, n_seqs), SP_THREADS, 0, stream>>>(a, w, slabs);
     space_run_scan_kernel<<<dim3((P * N + 4 * SP_THREADS - 1) / (4 * SP_THREADS), heads, n_seqs), SP_THREADS, 0, stream>>>(a, w);
 #define SPACE_OUT(PT)                                                                                                             \
     do {                                                                                                                          \

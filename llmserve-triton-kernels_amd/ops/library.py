@@ -1047,7 +1047,8 @@ def norm_store(q_out: torch.Tensor, proj: torch.Tensor, *, q_heads: int, k_heads
                slots: torch.Tensor | None = None, k_pool: torch.Tensor | None = None, v_pool: torch.Tensor | None = None,
                block_size: int = 0, freq: torch.Tensor | None = None, unit_norm: bool = False,
                angles: torch.Tensor | None = None, pairing: str = "half", norm_first: bool = False,
-               q_scale: torch.Tensor | None = None, values_from_keys: bool = False, joint: bool = False) -> torch.Tensor:
+               q_scale: torch.Tensor | None = None, values_from_keys: bool = False, joint: bool = False,
+               bias: torch.Tensor | None = None) -> torch.Tensor:
     """proj float32 [N, >= q_heads*dk + k_heads*dk + v_heads*dv] (q, k, v side by side; unit inner stride): with
     `freq` (float32 [rot_dims / 2]) the first rot_dims numbers of every head of q and k are first turned by the
     token's position (dimension i with dimension i + rot_dims / 2, angle position * freq[i]); `unit_norm`: every head
@@ -1060,8 +1061,9 @@ def norm_store(q_out: torch.Tensor, proj: torch.Tensor, *, q_heads: int, k_heads
     `angles` (rotary_angles(positions, freq), float32 [N, rot_dims / 2, 2]): the step's sines and cosines, which saves
     working them out (the same to the bit).  `q_scale` float32 [q_heads]: a factor per query head.  `values_from_keys`:
     proj holds no values; they are the keys as projected (v_heads = k_heads, dv = dk).  `joint`: one norm over all heads of
-    q and one over all heads of k (q_norm [q_heads * dk], k_norm [k_heads * dk]), before the rotation."""
-    dev = _dev(q_out, proj, q_norm, k_norm, positions, slots, k_pool, v_pool, freq, angles, q_scale)
+    q and one over all heads of k (q_norm [q_heads * dk], k_norm [k_heads * dk]), before the rotation; with it `bias`
+    (float32, a number per column of q, k and v) is added to proj first."""
+    dev = _dev(q_out, proj, q_norm, k_norm, positions, slots, k_pool, v_pool, freq, angles, q_scale, bias)
     n = proj.shape[0]
     if values_from_keys and (v_heads != k_heads or dv != dk):
         raise ValueError("values that are the keys have the keys' heads and size")
@@ -1089,6 +1091,10 @@ def norm_store(q_out: torch.Tensor, proj: torch.Tensor, *, q_heads: int, k_heads
             _f32(t, name, numbers if joint else dk)
     if joint and ((freq is not None and not norm_first) or max(q_heads, k_heads) * dk > 32768 or k_heads < 1):
         raise ValueError("one norm over all heads comes before the rotation and takes rows of up to 32,768 numbers")
+    if bias is not None:
+        if not joint:
+            raise ValueError("a bias goes with one norm over all heads")
+        _f32(bias, "bias", channels)
     if temp_every < 0:
         raise ValueError("temp_every must not be negative")
     if temp_every > 0:
@@ -1109,7 +1115,7 @@ def norm_store(q_out: torch.Tensor, proj: torch.Tensor, *, q_heads: int, k_heads
         _ptr(k_norm), c_float(eps), c_float(temp_coef), c_int(temp_every), _ptr(positions), _ptr(slots), _ptr(k_pool),
         _ptr(v_pool), c_int(n), c_int(q_heads), c_int(k_heads), c_int(dk), c_int(v_heads), c_int(dv), c_int(block_size),
         _ptr(freq), _ptr(angles), c_int(rot_dims), c_int(1 if unit_norm else 0), c_int(0 if _pairing(pairing) else 1),
-        c_int(1 if norm_first else 0), _ptr(q_scale), c_int(1 if values_from_keys else 0), c_int(1 if joint else 0), _stream(dev)),
+        c_int(1 if norm_first else 0), _ptr(q_scale), c_int(1 if values_from_keys else 0), c_int(1 if joint else 0), _ptr(bias), _stream(dev)),
         "norm_store")
     return q_out
 

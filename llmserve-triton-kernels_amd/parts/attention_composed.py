@@ -200,7 +200,7 @@ class ComposedAttention(Mixer):
             raise ValueError("a rotation and two score maps per head do not go together")
         if self.temp_every < 0:
             raise ValueError("query_temperature.every must be positive")
-        self.dist_bias = self.q_norm = self.k_norm = self.in_bias = None
+        self.dist_bias = self.q_norm = self.k_norm = self.in_bias = self.late_bias = None
         if self.num_heads % self.num_kv_heads:
             raise ValueError("num_heads must be a multiple of num_kv_heads")
         for name in ("window", "chunk"):
@@ -296,6 +296,8 @@ class ComposedAttention(Mixer):
             if self.output_gate:
                 biases.append(torch.zeros(self.gate_rows, dtype=biases[0].dtype, device=dev))
             self.in_bias = torch.cat(biases).contiguous()
+            if self.joint_norm:  # (added, in 32-bit, by the kernel that norms the projection)
+                self.late_bias, self.in_bias = torch.cat(biases[:len(kept)]).float().contiguous(), None
         if self.rot_dims:
             self.freq = torch.tensor(self.rot_freq, dtype=torch.float64).to(torch.float32).to(dev)
         if self.qk_norm_eps is not None and self.qk_norm_weight:
@@ -343,7 +345,7 @@ class ComposedAttention(Mixer):
                            block_size=paged.block_size, freq=self.freq,
                            unit_norm=self.qk_norm_eps is not None and not self.qk_norm_weight,
                            angles=step_angles(batch, self.freq, self.turn_key), pairing=self.pairing,
-                           norm_first=self.norm_first, q_scale=self.temp, values_from_keys=self.values_from_keys, joint=self.joint_norm)
+                           norm_first=self.norm_first, q_scale=self.temp, values_from_keys=self.values_from_keys, joint=self.joint_norm, bias=self.late_bias)
             out = torch.empty((proj.shape[0], heads * dv), dtype=x.dtype, device=x.device)
             self.attend(out, q, paged, view, batch, gate)
             return linear(out, self.o_weight, out_dtype=self.result_dtype)

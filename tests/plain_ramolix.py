@@ -157,7 +157,7 @@ def mamba2(h, t, p, m, eps):
     inner = H * P
     zxbcdt = h @ t[p + "in"].T
     z, xbc, dt = zxbcdt[:, :inner], zxbcdt[:, inner:2 * inner + 2 * G * N], zxbcdt[:, 2 * inner + 2 * G * N:]
-    xbc = silu(causal_conv(xbc, t[p + "conv"], t[p + "conv.b"]))
+    xbc = operand(silu(causal_conv(xbc, t[p + "conv"], t[p + "conv.b"])))
     x, B, C = xbc[:, :inner].view(T, H, P), xbc[:, inner:inner + G * N].view(T, G, N), xbc[:, inner + G * N:].view(T, G, N)
     dt = softplus(dt + t[p + "dt_bias"][None, :])
     y = state_space(x, B, C, dt, -torch.exp(t[p + "A_log"]), t[p + "D"]).reshape(T, inner)
